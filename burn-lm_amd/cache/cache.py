@@ -138,8 +138,13 @@ class KVGroup:
         """Pages wholly before the window of the *next* query are never read again."""
         if self.need.window <= 0:
             return 0
-        first_key = max(0, length_after - self.need.window + 1)  # oldest key the next token may see
+        first_key = max(0, length_after - self.need.window + 1)  # oldest key of the next token's window
         return first_key // self.page_size
+
+    @property
+    def kept_pages(self) -> int:
+        """The first pages of a sequence that stay although they lie before the window."""
+        return self.pages_for(self.need.keep_first) if self.need.window > 0 else 0
 
 
 class KVView:
@@ -246,7 +251,8 @@ class Cache:
         lib = _core.library()
         self._lib = lib
         self._h = lib.blm_cache_new(len(self.groups), _core.ints([g.n_pages for g in self.groups]),
-                                    _core.ints([g.need.window for g in self.groups]), page_size, max_seqs, max_context)
+                                    _core.ints([g.need.window for g in self.groups]), _core.ints([g.need.keep_first for g in self.groups]),
+                                    page_size, max_seqs, max_context)
         if not self._h:
             raise CacheError("the native cache core refused these sizes")
         for gi, g in enumerate(self.groups):
@@ -260,7 +266,7 @@ class Cache:
         total = 0
         for v in (c for v in self.views for c in (v if isinstance(v, tuple) else (v,))):
             if isinstance(v, KVView):
-                keys = min(length, v.need.window) if v.need.window > 0 else length
+                keys = min(length, v.need.window + v.need.keep_first) if v.need.window > 0 else length
                 total += (v.need.n_kv_heads * v.need.head_dim + v.need.v_heads * v.need.v_dim) * keys * v.k.element_size()
             elif with_state and isinstance(v, StateView):      # fixed-size state is read and written once a step
                 total += 2 * v.tensor[0].numel() * v.tensor.element_size()

@@ -8,7 +8,7 @@ from typing import List, Sequence
 
 from ..csrc import build as _build
 
-HOST_ABI = 4
+HOST_ABI = 5
 OK, E_FULL, E_OVERFLOW, E_USAGE = 0, 1, 2, 3
 
 _lib = None
@@ -20,7 +20,7 @@ _SIGNATURES = {
     "blm_pool_new": ([_int], _ptr), "blm_pool_free": ([_ptr], None), "blm_pool_n_free": ([_ptr], _int),
     "blm_pool_take": ([_ptr, _int, _ints], _int), "blm_pool_give": ([_ptr, _int, _ints], _int),
     "blm_pool_free_list": ([_ptr, _ints], _int), "blm_pool_is_out": ([_ptr, _int], _int),
-    "blm_cache_new": ([_int, _ints, _ints, _int, _int, _int], _ptr), "blm_cache_free": ([_ptr], None),
+    "blm_cache_new": ([_int, _ints, _ints, _ints, _int, _int, _int], _ptr), "blm_cache_free": ([_ptr], None),
     "blm_cache_open": ([_ptr, _ints], _int), "blm_cache_close": ([_ptr, _int], _int),
     "blm_cache_length": ([_ptr, _int], _int), "blm_cache_reserve": ([_ptr, _int, _ints, _ints, _ints], _int),
     "blm_cache_advance": ([_ptr, _int, _int], _int), "blm_cache_table_len": ([_ptr, _int, _int], _int),

@@ -18,6 +18,8 @@
 // Decode:  they are the query heads that share a key-value head, for one token; the key range is
 //          cut into splits that are merged afterwards (float partial results).
 // Visibility: query at position p sees keys j <= p of its sequence and, with a window w, p - j < w.
+// EXT kernels also take: keep_first, the number of a sequence's first keys that stay visible before the window (the
+// pages that hold them are walked ahead of the window's), and cap, scores s <- cap * tanh(s / cap) (0: as they are).
 #include <stdlib.h>
 
 #include <type_traits>
@@ -160,10 +162,38 @@ struct DirectStage {
   }
 };
 
-template <int HD, bool FULL, class PAGE>
+// What an EXT kernel adds to the scores: s2 = cap2 * tanh(s * to_half) as exponents of two, with tanh(z) written as
+// 1 - 2 / (1 + 2^(2 z log2 e)): cap2 = cap * log2(e), to_half = 2 * log2(e) * scale / cap.  cap2 = 0: no cap.
+struct AmExt {
+  int keep_first;
+  float cap2, to_half;
+};
+__device__ __forceinline__ AmExt am_ext(int keep_first, float cap, float scale) {
+  AmExt x;
+  x.keep_first = keep_first;
+  x.cap2 = cap * 1.4426950408889634f;
+  x.to_half = cap > 0.f ? 2.0f * 1.4426950408889634f * scale / cap : 0.f;
+  return x;
+}
+__device__ __forceinline__ float am_capped(float s, const AmExt& x) {
+  return x.cap2 * (1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s * x.to_half)));
+}
+// The pages a query tile walks: those of the first keys that stay visible, then those from `first` to `last`.  EXT:
+// otherwise the window's alone.
+struct AmWalk {
+  int kept, first, last;
+  __device__ __forceinline__ int count() const { return kept + last - first + 1; }
+  __device__ __forceinline__ int page(int x) const { return x < kept ? x : first + x - kept; }
+};
+template <bool EXT>
+__device__ __forceinline__ AmWalk am_walk(int first, int last, int keep_first) {
+  return AmWalk{EXT ? min((keep_first + AM_PAGE - 1) / AM_PAGE, first) : 0, first, last};
+}
+
+template <int HD, bool FULL, class PAGE, bool EXT>
 __device__ __forceinline__ void attn_page(const bf16* __restrict__ kp, const bf16* __restrict__ vp,
                                           const uint4* qf, int key0, int qpos, int lo, int max_key, float scale2,
-                                          float& m, f32x4_t& l, f32x4_t* o) {
+                                          float& m, f32x4_t& l, f32x4_t* o, const AmExt& ext) {
   constexpr int KS = (HD + 31) / 32;
   constexpr int DT = (HD + 15) / 16;
   const int lane = threadIdx.x & (BLM_WAVE - 1);
@@ -188,13 +218,17 @@ __device__ __forceinline__ void attn_page(const bf16* __restrict__ kp, const bf1
     for (int ks = 0; ks < KS; ++ks)
       acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kf[t][ks]),
                                                     __builtin_bit_cast(bf16x8_t, qf[ks]), acc, 0, 0, 0);
+    if (EXT && ext.cap2 > 0.f) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) acc[r] = am_capped(acc[r], ext);
+    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       if (FULL) {
         s[t][r] = acc[r];
       } else {
         const int kj = key0 + am_key_of(t, kg * 4 + r);
-        s[t][r] = (kj <= qpos && kj >= lo) ? acc[r] : -INFINITY;
+        s[t][r] = (kj <= qpos && (kj >= lo || (EXT && kj < ext.keep_first))) ? acc[r] : -INFINITY;
       }
     }
   }
@@ -301,13 +335,13 @@ __device__ __forceinline__ void load_q(const bf16* qrow, uint4* qf) {
 // while the current one is used) and each wavefront takes its MFMA fragments from there; rows are
 // padded by 16 bytes so that the fragment reads do not collide.
 // ---------------------------------------------------------------------------------------
-template <int HD>
+template <int HD, bool EXT>
 __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 4 : (HD <= 128 ? 2 : 1), HD <= 64 ? 8 : (HD <= 128 ? 2 : 1))))
     attn_prefill_mfma_kernel(const bf16* __restrict__ q, int q_row_stride, bf16* __restrict__ out,
                              const int* __restrict__ positions, const int* __restrict__ cu_seqlens,
                              const int* __restrict__ block_table, int table_width,
                              const bf16* __restrict__ kcache, const bf16* __restrict__ vcache, int nh, int nkv,
-                             float scale, int window, const float* __restrict__ sinks) {
+                             float scale, int window, const float* __restrict__ sinks, int keep_first, float cap) {
   constexpr int KS = (HD + 31) / 32;
   constexpr int DT = (HD + 15) / 16;
   // Head sizes 64 and 128: a page comes straight from global memory into shared memory, its rows'
@@ -362,6 +396,8 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
   const int blk_qlast = positions[row_begin + min(qt_hi * 16 + 15, n_b - 1)];
   const int blk_first = ((window > 0 && blk_qfirst - window + 1 > 0) ? blk_qfirst - window + 1 : 0) / AM_PAGE;
   const int blk_last = blk_qlast / AM_PAGE;
+  const AmWalk walk = am_walk<EXT>(blk_first, blk_last, keep_first);
+  const int n_pages = walk.count();
 
   uint4 qf[KS];
   load_q<HD>(q + (size_t)row * q_row_stride + (size_t)head * HD, qf);
@@ -372,9 +408,10 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
   f32x4_t o[DT];
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) o[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  const float scale2 = scale * 1.4426950408889634f;
+  const AmExt ext = am_ext(EXT ? keep_first : 0, EXT ? cap : 0.f, scale);
+  const float scale2 = (EXT && cap > 0.f) ? 1.0f : scale * 1.4426950408889634f;      // capped scores are exponents of two already
   PageNumbers pages{block_table + (size_t)b * table_width, table_width, 0, 0};
-  pages.load(blk_first);
+  pages.load(walk.page(0));
 
   u32x4_t kreg[PER_THREAD], vreg[PER_THREAD];
 #define AM_FETCH(pi)                                                                          \
@@ -399,31 +436,31 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
     }                                                                                                           \
   }
 #define AM_USE(buf)                                                                                           \
-  if (pi >= my_first && pi <= my_last) {                                                                        \
+  if (pi <= my_last && (pi >= my_first || (EXT && pi * AM_PAGE < keep_first))) {                                \
     const int key0 = pi * AM_PAGE;                                                                              \
     /* pages wholly inside every query's range need no mask */                                                  \
-    if (key0 + AM_PAGE - 1 <= qpos_first && key0 >= lo_last)                                                    \
-      attn_page<HD, true, PAGE>(k_lds[buf], v_lds[buf], qf, key0, qpos, lo, seq_last, scale2, m, lsum, o);  \
+    if (key0 + AM_PAGE - 1 <= qpos_first && (key0 >= lo_last || (EXT && key0 + AM_PAGE <= keep_first)))         \
+      attn_page<HD, true, PAGE, EXT>(k_lds[buf], v_lds[buf], qf, key0, qpos, lo, seq_last, scale2, m, lsum, o, ext);  \
     else                                                                                                        \
-      attn_page<HD, false, PAGE>(k_lds[buf], v_lds[buf], qf, key0, qpos, lo, seq_last, scale2, m, lsum, o); \
+      attn_page<HD, false, PAGE, EXT>(k_lds[buf], v_lds[buf], qf, key0, qpos, lo, seq_last, scale2, m, lsum, o, ext); \
   }
   if constexpr (DIRECT) {
     DirectStage<DIRECT ? HD : 64, TileOrder16> stage;
     stage.init(k_lds[0], v_lds[0]);
     auto fetch = [&](int pi, int buf) { stage.fetch(kcache, vcache, ((size_t)pages.at(pi) * nkv + kvh) * AM_PAGE * HD, buf); };
-    fetch(blk_first, 0);
+    fetch(walk.page(0), 0);
     am_pin<KS>(qf);   // see below
     AM_WAIT_LOADS();
     __syncthreads();
-    for (int pi = blk_first; pi <= blk_last; ++pi) {
-      const int cur = (pi - blk_first) & 1;
-      if (pi < blk_last) fetch(pi + 1, cur ^ 1);   // into the other buffer, which nobody reads now
+    for (int x = 0; x < n_pages; ++x) {
+      const int cur = x & 1, pi = walk.page(x);
+      if (x + 1 < n_pages) fetch(walk.page(x + 1), cur ^ 1);   // into the other buffer, which nobody reads now
       AM_USE(cur)
       AM_WAIT_LOADS();     // the compiler does not know of these loads: the wait is the program's own
       __syncthreads();     // the next page is in place, and everybody is done with this one
     }
   } else {
-  AM_FETCH(blk_first);
+  AM_FETCH(walk.page(0));
   // The query fragments have arrived before the loop starts.  Left alone, the compiler moves their
   // loads down to the loop's entry, and since its count of outstanding loads is merged over the loop's
   // paths, it then waits in front of the first product of every page for all loads, the page it has
@@ -432,19 +469,20 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
   if (NBUF == 2) {
     AM_STAGE(0)
     __syncthreads();
-    for (int pi = blk_first; pi <= blk_last; ++pi) {
-      const int cur = (pi - blk_first) & 1;
-      if (pi < blk_last) AM_FETCH(pi + 1);   // travels while this page is used
+    for (int x = 0; x < n_pages; ++x) {
+      const int cur = x & 1, pi = walk.page(x);
+      if (x + 1 < n_pages) AM_FETCH(walk.page(x + 1));   // travels while this page is used
       AM_USE(cur)
-      if (pi < blk_last) { AM_STAGE(cur ^ 1) }   // the other buffer: nobody reads it now
+      if (x + 1 < n_pages) { AM_STAGE(cur ^ 1) }   // the other buffer: nobody reads it now
       __syncthreads();   // the next page is in place, and everybody is done with this one
     }
   } else {
-    for (int pi = blk_first; pi <= blk_last; ++pi) {
+    for (int x = 0; x < n_pages; ++x) {
+      const int pi = walk.page(x);
       __syncthreads();   // the page before has been used by every wavefront
       AM_STAGE(0)
       __syncthreads();
-      if (pi < blk_last) AM_FETCH(pi + 1);   // travels while this page is used
+      if (x + 1 < n_pages) AM_FETCH(walk.page(x + 1));   // travels while this page is used
       AM_USE(0)
     }
   }
@@ -518,10 +556,10 @@ __device__ __forceinline__ float am_dot2_ones(uint32_t pair, float acc) {
 // Half `half` of a page (32 keys from key0) for one wavefront: the softmax state advances once per 32
 // keys, so only 16 scores per lane are alive at a time.  kp, vp: the staged page; FRAG: where its
 // fragments lie.  max_key: the last key that the cache holds data for (see attn_page).
-template <int HD, bool FULL, class FRAG>
+template <int HD, bool FULL, class FRAG, bool EXT>
 __device__ __forceinline__ void attn_half32(const bf16* __restrict__ kp, const bf16* __restrict__ vp, const uint4* qf,
                                             int half, int key0, int qpos, int lo, int max_key, float scale2, float& m,
-                                            float& l, f32x16_t* o) {
+                                            float& l, f32x16_t* o, const AmExt& ext) {
   constexpr int KS = HD / 16, RT = HD / 32;
   const int lane = threadIdx.x & (BLM_WAVE - 1);
   const int j = lane & 31, hb = lane >> 5;
@@ -533,11 +571,15 @@ __device__ __forceinline__ void attn_half32(const bf16* __restrict__ kp, const b
     const uint4 kf = *reinterpret_cast<const uint4*>(kp + FRAG::k(half * 32 + j, ks, hb));
     s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, kf), __builtin_bit_cast(bf16x8_t, qf[ks]), s, 0, 0, 0);
   }
+  if (EXT && ext.cap2 > 0.f) {
+#pragma unroll
+    for (int v = 0; v < 16; ++v) s[v] = am_capped(s[v], ext);
+  }
   if (!FULL) {
 #pragma unroll
     for (int v = 0; v < 16; ++v) {
       const int kj = key0 + TileOrder32::key_of(8 * (v >> 2) + 4 * hb + (v & 3));
-      s[v] = (kj <= qpos && kj >= lo) ? s[v] : -INFINITY;
+      s[v] = (kj <= qpos && (kj >= lo || (EXT && kj < ext.keep_first))) ? s[v] : -INFINITY;
     }
   }
   float mx = blm_max(s[0], s[1]);
@@ -585,25 +627,25 @@ __device__ __forceinline__ void attn_half32(const bf16* __restrict__ kp, const b
 }
 
 // tile_last: the last key that any query of the tile sees
-template <int HD, bool FULL, class FRAG>
+template <int HD, bool FULL, class FRAG, bool EXT>
 __device__ __forceinline__ void attn_page32(const bf16* __restrict__ kp, const bf16* __restrict__ vp, const uint4* qf,
                                             int key0, int qpos, int lo, int tile_last, int max_key, float scale2, float& m,
-                                            float& l, f32x16_t* o) {
-  attn_half32<HD, FULL, FRAG>(kp, vp, qf, 0, key0, qpos, lo, max_key, scale2, m, l, o);
+                                            float& l, f32x16_t* o, const AmExt& ext) {
+  attn_half32<HD, FULL, FRAG, EXT>(kp, vp, qf, 0, key0, qpos, lo, max_key, scale2, m, l, o, ext);
   // the second half of a page on the diagonal may lie wholly behind the tile's last query
   if (FULL || key0 + 32 <= tile_last)
-    attn_half32<HD, FULL, FRAG>(kp, vp, qf, 1, key0 + 32, qpos, lo, max_key, scale2, m, l, o);
+    attn_half32<HD, FULL, FRAG, EXT>(kp, vp, qf, 1, key0 + 32, qpos, lo, max_key, scale2, m, l, o, ext);
 }
 
 // grid (ceil(G * q_tiles32 / 4), kv heads, sequences); the block order and the page staging are those
 // of the 16-query kernel above
-template <int HD>
+template <int HD, bool EXT>
 __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 4 : 2, HD <= 64 ? 4 : 2)))
     attn_prefill32_kernel(const bf16* __restrict__ q, int q_row_stride, bf16* __restrict__ out,
                           const int* __restrict__ positions, const int* __restrict__ cu_seqlens,
                           const int* __restrict__ block_table, int table_width,
                           const bf16* __restrict__ kcache, const bf16* __restrict__ vcache, int nh, int nkv,
-                          float scale, int window, const float* __restrict__ sinks) {
+                          float scale, int window, const float* __restrict__ sinks, int keep_first, float cap) {
   static_assert(HD % 32 == 0 && HD <= 128, "32-query prefill: head sizes 32, 64, 96, 128");
   constexpr int KS = HD / 16, RT = HD / 32, QT = 32;
   constexpr bool DIRECT = HD == 64 || HD == 128;   // as in the 16-query kernel
@@ -648,6 +690,8 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
   const int blk_qlast = positions[row_begin + min(qt_hi * QT + QT - 1, n_b - 1)];
   const int blk_first = ((window > 0 && blk_qfirst - window + 1 > 0) ? blk_qfirst - window + 1 : 0) / AM_PAGE;
   const int blk_last = blk_qlast / AM_PAGE;
+  const AmWalk walk = am_walk<EXT>(blk_first, blk_last, keep_first);
+  const int n_pages = walk.count();
 
   uint4 qf[KS];
   {
@@ -662,9 +706,10 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
   for (int rt = 0; rt < RT; ++rt)
 #pragma unroll
     for (int v = 0; v < 16; ++v) o[rt][v] = 0.f;
-  const float scale2 = scale * 1.4426950408889634f;
+  const AmExt ext = am_ext(EXT ? keep_first : 0, EXT ? cap : 0.f, scale);
+  const float scale2 = (EXT && cap > 0.f) ? 1.0f : scale * 1.4426950408889634f;      // capped scores are exponents of two already
   PageNumbers pages{block_table + (size_t)b * table_width, table_width, 0, 0};
-  pages.load(blk_first);
+  pages.load(walk.page(0));
 
   u32x4_t kreg[PER_THREAD], vreg[PER_THREAD];
 #define AP_FETCH(pi)                                                                          \
@@ -689,38 +734,38 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
     }                                                                                                           \
   }
 #define AP_USE(buf)                                                                                           \
-  if (pi >= my_first && pi <= my_last) {                                                                        \
+  if (pi <= my_last && (pi >= my_first || (EXT && pi * AM_PAGE < keep_first))) {                                \
     const int key0 = pi * AM_PAGE;                                                                              \
-    if (key0 + AM_PAGE - 1 <= qpos_first && key0 >= lo_last)                                                    \
-      attn_page32<HD, true, FRAG>(k_lds[buf], v_lds[buf], qf, key0, qpos, lo, qpos_last, seq_last, scale2, m, lsum, o);  \
+    if (key0 + AM_PAGE - 1 <= qpos_first && (key0 >= lo_last || (EXT && key0 + AM_PAGE <= keep_first)))         \
+      attn_page32<HD, true, FRAG, EXT>(k_lds[buf], v_lds[buf], qf, key0, qpos, lo, qpos_last, seq_last, scale2, m, lsum, o, ext);  \
     else                                                                                                        \
-      attn_page32<HD, false, FRAG>(k_lds[buf], v_lds[buf], qf, key0, qpos, lo, qpos_last, seq_last, scale2, m, lsum, o); \
+      attn_page32<HD, false, FRAG, EXT>(k_lds[buf], v_lds[buf], qf, key0, qpos, lo, qpos_last, seq_last, scale2, m, lsum, o, ext); \
   }
   if constexpr (DIRECT) {
     DirectStage<DIRECT ? HD : 64, TileOrder32> stage;
     stage.init(k_lds[0], v_lds[0]);
     auto fetch = [&](int pi, int buf) { stage.fetch(kcache, vcache, ((size_t)pages.at(pi) * nkv + kvh) * AM_PAGE * HD, buf); };
-    fetch(blk_first, 0);
+    fetch(walk.page(0), 0);
     am_pin<HD / 16>(qf);   // as in the 16-query kernel
     AM_WAIT_LOADS();
     __syncthreads();
-    for (int pi = blk_first; pi <= blk_last; ++pi) {
-      const int cur = (pi - blk_first) & 1;
-      if (pi < blk_last) fetch(pi + 1, cur ^ 1);   // into the other buffer, which nobody reads now
+    for (int x = 0; x < n_pages; ++x) {
+      const int cur = x & 1, pi = walk.page(x);
+      if (x + 1 < n_pages) fetch(walk.page(x + 1), cur ^ 1);   // into the other buffer, which nobody reads now
       AP_USE(cur)
       AM_WAIT_LOADS();
       __syncthreads();     // the next page is in place, and everybody is done with this one
     }
   } else {
-    AP_FETCH(blk_first);
+    AP_FETCH(walk.page(0));
     am_pin<HD / 16>(qf);   // as in the 16-query kernel
     AP_STAGE(0)
     __syncthreads();
-    for (int pi = blk_first; pi <= blk_last; ++pi) {
-      const int cur = (pi - blk_first) & 1;
-      if (pi < blk_last) AP_FETCH(pi + 1);   // travels while this page is used
+    for (int x = 0; x < n_pages; ++x) {
+      const int cur = x & 1, pi = walk.page(x);
+      if (x + 1 < n_pages) AP_FETCH(walk.page(x + 1));   // travels while this page is used
       AP_USE(cur)
-      if (pi < blk_last) { AP_STAGE(cur ^ 1) }   // the other buffer: nobody reads it now
+      if (x + 1 < n_pages) { AP_STAGE(cur ^ 1) }   // the other buffer: nobody reads it now
       __syncthreads();   // the next page is in place, and everybody is done with this one
     }
   }
@@ -753,13 +798,14 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
 //   part_o [T, nh, splits, HD] float, part_ml [T, nh, splits, 2] float,
 // merged by whichever split of a (token, head tile) finishes last
 // ---------------------------------------------------------------------------------------
-template <int HD>
+template <int HD, bool EXT>
 __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE)
     attn_decode_mfma_kernel(const bf16* __restrict__ q, int q_row_stride, const int* __restrict__ positions,
                             const int* __restrict__ token_seq, const int* __restrict__ block_table,
                             int table_width, const bf16* __restrict__ kcache, const bf16* __restrict__ vcache,
                             int nh, int nkv, float scale, int window, int n_splits, float* part_o,
-                            float* part_ml, int* arrivals, bf16* out, const float* __restrict__ sinks) {
+                            float* part_ml, int* arrivals, bf16* out, const float* __restrict__ sinks, int keep_first,
+                            float cap) {
   constexpr int KS = (HD + 31) / 32;
   constexpr int DT = (HD + 15) / 16;
   // Every wavefront brings its pages through a staging area of its own in shared memory: whole
@@ -801,15 +847,17 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE)
   if (b >= 0) {
     const int pos = positions[t];
     const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
-    const int first_page = lo / AM_PAGE, last_page = pos / AM_PAGE;
-    const int per_split = (last_page - first_page + 1 + n_splits - 1) / n_splits;
-    const int p_begin = first_page + split * per_split;
-    const int p_end = min(last_page + 1, p_begin + per_split);
+    const AmWalk walk = am_walk<EXT>(lo / AM_PAGE, pos / AM_PAGE, keep_first);
+    const AmExt ext = am_ext(EXT ? keep_first : 0, EXT ? cap : 0.f, scale);
+    const int n_walk = walk.count();
+    const int per_split = (n_walk + n_splits - 1) / n_splits;
+    const int p_begin = split * per_split;      // places of the walk
+    const int p_end = min(n_walk, p_begin + per_split);
     PageNumbers pages{block_table + (size_t)b * table_width, table_width, 0, 0};
-    if (p_begin < p_end) pages.load(p_begin);
+    if (p_begin < p_end) pages.load(walk.page(p_begin));
     uint4 qf[KS];
     load_q<HD>(q + (size_t)t * q_row_stride + (size_t)head * HD, qf);
-    const float scale2 = scale * 1.4426950408889634f;
+    const float scale2 = (EXT && cap > 0.f) ? 1.0f : scale * 1.4426950408889634f;
     u32x4_t kreg[PER_LANE], vreg[PER_LANE];
 #define AD_FETCH(pi)                                                                          \
   {                                                                                           \
@@ -828,17 +876,17 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE)
     const int vr = j / (AM_PAGE / 8), vc = j - vr * (AM_PAGE / 8); /* value row (a dim), 16-byte column */      \
     *reinterpret_cast<u32x4_t*>(v_lds + vr * VSTR + vc * 8) = vreg[i];                                          \
   }
-    int pi = p_begin + wave;
-    if (pi < p_end) AD_FETCH(pi);
+    int x = p_begin + wave;
+    if (x < p_end) AD_FETCH(walk.page(x));
     am_pin<KS>(qf);   // arrived before the loop, so that no page's first product waits for the page just asked for
-    for (; pi < p_end; pi += AM_WAVES) {
+    for (; x < p_end; x += AM_WAVES) {
       AD_STAGE()
-      if (pi + AM_WAVES < p_end) AD_FETCH(pi + AM_WAVES);   // travels while this page is used
-      const int key0 = pi * AM_PAGE;
-      if (key0 + AM_PAGE - 1 <= pos && key0 >= lo)
-        attn_page<HD, true, PaddedPage<HD>>(k_lds, v_lds, qf, key0, pos, lo, pos, scale2, m, lsum, o);
+      if (x + AM_WAVES < p_end) AD_FETCH(walk.page(x + AM_WAVES));   // travels while this page is used
+      const int key0 = walk.page(x) * AM_PAGE;
+      if (key0 + AM_PAGE - 1 <= pos && (key0 >= lo || (EXT && key0 + AM_PAGE <= keep_first)))
+        attn_page<HD, true, PaddedPage<HD>, EXT>(k_lds, v_lds, qf, key0, pos, lo, pos, scale2, m, lsum, o, ext);
       else
-        attn_page<HD, false, PaddedPage<HD>>(k_lds, v_lds, qf, key0, pos, lo, pos, scale2, m, lsum, o);
+        attn_page<HD, false, PaddedPage<HD>, EXT>(k_lds, v_lds, qf, key0, pos, lo, pos, scale2, m, lsum, o, ext);
     }
 #undef AD_FETCH
 #undef AD_STAGE
@@ -956,13 +1004,14 @@ extern "C" int blm_attn_prefill_mfma(const void* q, int q_row_stride, void* out,
                                      const int* positions, const int* cu_seqlens, const int* block_table,
                                      int table_width, const void* kcache, const void* vcache, int page_size,
                                      int n_seqs, int max_new, int nh, int nkv, int hd, float scale, int window,
-                                     int queries, const float* sinks, hipStream_t stream) {
+                                     int queries, const float* sinks, int keep_first, float cap, hipStream_t stream) {
   BLM_REQUIRE(n_seqs > 0 && n_seqs <= 65535 && max_new > 0 && nh > 0 && nkv > 0 && nkv <= 65535 && nh % nkv == 0,
               "attn_prefill_mfma: bad sizes seqs=%d max_new=%d heads=%d kv_heads=%d", n_seqs, max_new, nh, nkv);
   BLM_REQUIRE(blm_attn_prefill_mfma_supported(act_dtype, hd, page_size),
               "attn_prefill_mfma: needs bfloat16, pages of 64 and a head_dim that is a multiple of 16 up to 128, or 256 "
               "(got dtype %d, page %d, head_dim %d)", act_dtype, page_size, hd);
-  BLM_REQUIRE(table_width > 0 && window >= 0, "attn_prefill_mfma: bad geometry");
+  BLM_REQUIRE(table_width > 0 && window >= 0 && keep_first >= 0 && cap >= 0.f, "attn_prefill_mfma: bad geometry");
+  const bool extended = keep_first > 0 || cap > 0.f;
   BLM_REQUIRE(scale > 0.f, "attn_prefill_mfma: the score scale must be positive (got %g)", (double)scale);
   BLM_REQUIRE(q_row_stride % 8 == 0 && ((uintptr_t)q % 16) == 0 && ((uintptr_t)out % 8) == 0,
               "attn_prefill_mfma: q rows must be 16-byte aligned");
@@ -982,9 +1031,14 @@ extern "C" int blm_attn_prefill_mfma(const void* q, int q_row_stride, void* out,
     dim3 grid32((unsigned)((units32 + AM_WAVES - 1) / AM_WAVES), nkv, n_seqs), block32(AM_WAVES * BLM_WAVE);
 #define BLM_AP32(HD)                                                                                             \
   case HD:                                                                                                       \
-    hipLaunchKernelGGL((attn_prefill32_kernel<HD>), grid32, block32, 0, stream, (const bf16*)q, q_row_stride,     \
-                       (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,          \
-                       (const bf16*)vcache, nh, nkv, scale, window, sinks);                                       \
+    if (extended)                                                                                                \
+      hipLaunchKernelGGL((attn_prefill32_kernel<HD, true>), grid32, block32, 0, stream, (const bf16*)q, q_row_stride, \
+                         (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
+                         (const bf16*)vcache, nh, nkv, scale, window, sinks, keep_first, cap);                    \
+    else                                                                                                         \
+      hipLaunchKernelGGL((attn_prefill32_kernel<HD, false>), grid32, block32, 0, stream, (const bf16*)q, q_row_stride, \
+                         (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
+                         (const bf16*)vcache, nh, nkv, scale, window, sinks, 0, 0.f);                             \
     break
     switch (hd) {
       BLM_AP32(32); BLM_AP32(64); BLM_AP32(96); BLM_AP32(128);
@@ -997,9 +1051,14 @@ extern "C" int blm_attn_prefill_mfma(const void* q, int q_row_stride, void* out,
   dim3 grid((unsigned)((units + AM_WAVES - 1) / AM_WAVES), nkv, n_seqs), block(AM_WAVES * BLM_WAVE);
 #define BLM_AP(HD)                                                                                               \
   case HD:                                                                                                       \
-    hipLaunchKernelGGL((attn_prefill_mfma_kernel<HD>), grid, block, 0, stream, (const bf16*)q, q_row_stride,      \
-                       (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,          \
-                       (const bf16*)vcache, nh, nkv, scale, window, sinks);                                       \
+    if (extended)                                                                                                \
+      hipLaunchKernelGGL((attn_prefill_mfma_kernel<HD, true>), grid, block, 0, stream, (const bf16*)q, q_row_stride, \
+                         (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
+                         (const bf16*)vcache, nh, nkv, scale, window, sinks, keep_first, cap);                    \
+    else                                                                                                         \
+      hipLaunchKernelGGL((attn_prefill_mfma_kernel<HD, false>), grid, block, 0, stream, (const bf16*)q, q_row_stride, \
+                         (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
+                         (const bf16*)vcache, nh, nkv, scale, window, sinks, 0, 0.f);                             \
     break
   switch (hd) {
     BLM_AP(16); BLM_AP(32); BLM_AP(48); BLM_AP(64); BLM_AP(80); BLM_AP(96); BLM_AP(112); BLM_AP(128); BLM_AP(256);
@@ -1016,7 +1075,8 @@ extern "C" int blm_attn_decode(const void* q, int q_row_stride, void* out, int a
                                const int* token_seq, const int* block_table, int table_width, const void* kcache,
                                const void* vcache, int page_size, int T, int nh, int nkv, int hd, float scale,
                                int window, int n_splits, float* part_o, float* part_ml, int* arrivals,
-                               const float* sinks, hipStream_t stream) {
+                               const float* sinks, int keep_first, float cap, hipStream_t stream) {
+  BLM_REQUIRE(keep_first >= 0 && cap >= 0.f, "attn_decode: keep_first %d or cap %g is negative", keep_first, (double)cap);
   BLM_REQUIRE(T > 0 && T <= 65535 && nh > 0 && nkv > 0 && nh % nkv == 0,
               "attn_decode: bad sizes T=%d heads=%d kv_heads=%d", T, nh, nkv);
   BLM_REQUIRE(blm_attn_decode_supported(act_dtype, hd, page_size),
@@ -1034,9 +1094,14 @@ extern "C" int blm_attn_decode(const void* q, int q_row_stride, void* out, int a
   dim3 grid(n_splits, nkv * gtiles, T), block(AM_WAVES * BLM_WAVE);
 #define BLM_AD(HD)                                                                                                 \
   case HD:                                                                                                         \
-    hipLaunchKernelGGL((attn_decode_mfma_kernel<HD>), grid, block, 0, stream, (const bf16*)q, q_row_stride,         \
-                       positions, token_seq, block_table, table_width, (const bf16*)kcache, (const bf16*)vcache,    \
-                       nh, nkv, scale, window, n_splits, part_o, part_ml, arrivals, (bf16*)out, sinks);             \
+    if (keep_first > 0 || cap > 0.f)                                                                               \
+      hipLaunchKernelGGL((attn_decode_mfma_kernel<HD, true>), grid, block, 0, stream, (const bf16*)q, q_row_stride, \
+                         positions, token_seq, block_table, table_width, (const bf16*)kcache, (const bf16*)vcache,  \
+                         nh, nkv, scale, window, n_splits, part_o, part_ml, arrivals, (bf16*)out, sinks, keep_first, cap); \
+    else                                                                                                           \
+      hipLaunchKernelGGL((attn_decode_mfma_kernel<HD, false>), grid, block, 0, stream, (const bf16*)q, q_row_stride, \
+                         positions, token_seq, block_table, table_width, (const bf16*)kcache, (const bf16*)vcache,  \
+                         nh, nkv, scale, window, n_splits, part_o, part_ml, arrivals, (bf16*)out, sinks, 0, 0.f);   \
     break
   switch (hd) { BLM_AD(16); BLM_AD(32); BLM_AD(48); BLM_AD(64); BLM_AD(80); BLM_AD(96); BLM_AD(112); BLM_AD(128); }
 #undef BLM_AD

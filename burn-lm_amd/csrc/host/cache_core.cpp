@@ -98,7 +98,7 @@ extern "C" int blm_pool_is_out(const BlmPool* p, int page) {
 
 // ---- cache ----------------------------------------------------------------------------------------
 struct Group {
-  int window;
+  int window, keep_first;
   BlmPool pool;
   std::vector<std::vector<int>> tables;   // per slot: page of each page index, -1 once released
 };
@@ -119,10 +119,13 @@ static inline int first_needed_page(const BlmCache& c, const Group& g, int lengt
   return first_key / c.page_size;
 }
 
+// pages that hold a sequence's first keys where those stay beside a window
+static inline int kept_pages(const BlmCache& c, const Group& g) { return g.window > 0 ? pages_for(c, g.keep_first) : 0; }
+
 static inline bool is_open(const BlmCache& c, int slot) { return slot >= 0 && slot < c.max_seqs && c.length[slot] >= 0; }
 
-extern "C" BlmCache* blm_cache_new(int n_groups, const int* n_pages, const int* windows, int page_size, int max_seqs,
-                                   int max_context) {
+extern "C" BlmCache* blm_cache_new(int n_groups, const int* n_pages, const int* windows, const int* keep_first, int page_size,
+                                   int max_seqs, int max_context) {
   if (n_groups < 0 || page_size <= 0 || max_seqs <= 0 || max_context <= 0) return nullptr;
   BlmCache* c = new BlmCache();
   c->page_size = page_size;
@@ -131,6 +134,7 @@ extern "C" BlmCache* blm_cache_new(int n_groups, const int* n_pages, const int* 
   c->groups.resize(n_groups);
   for (int g = 0; g < n_groups; ++g) {
     c->groups[g].window = windows[g];
+    c->groups[g].keep_first = keep_first ? std::max(0, keep_first[g]) : 0;
     pool_init(c->groups[g].pool, n_pages[g]);
     c->groups[g].tables.resize(max_seqs);
   }
@@ -215,7 +219,7 @@ extern "C" int blm_cache_advance(BlmCache* c, int slot, int n) {
   for (Group& g : c->groups) {
     std::vector<int>& table = g.tables[slot];
     const int first = std::min<int>(first_needed_page(*c, g, c->length[slot]), (int)table.size());
-    for (int i = 0; i < first; ++i) {
+    for (int i = kept_pages(*c, g); i < first; ++i) {
       if (table[i] >= 0) {
         const int rc = pool_give(g.pool, 1, &table[i]);
         if (rc) return rc;

@@ -10,7 +10,7 @@
 extern "C" {
 #endif
 
-#define BLM_HOST_ABI 4
+#define BLM_HOST_ABI 5
 
 #define BLM_OK 0
 #define BLM_E_FULL 1      // no free slot, or not enough free pages
@@ -32,10 +32,11 @@ int blm_pool_is_out(const BlmPool*, int page);
 
 // ---- the cache's bookkeeping ----------------------------------------------------------------
 // Groups of layers with the same need share pages; group g has n_pages[g] pages of page_size
-// tokens and keeps the last windows[g] keys of a sequence (0: all of them).
+// tokens and keeps the last windows[g] keys of a sequence (0: all of them) and, beside a window, the
+// first keep_first[g] keys (null: none).
 typedef struct BlmCache BlmCache;
-BlmCache* blm_cache_new(int n_groups, const int* n_pages, const int* windows, int page_size, int max_seqs,
-                        int max_context);
+BlmCache* blm_cache_new(int n_groups, const int* n_pages, const int* windows, const int* keep_first, int page_size,
+                        int max_seqs, int max_context);
 void blm_cache_free(BlmCache*);
 int blm_cache_open(BlmCache*, int* slot);
 int blm_cache_close(BlmCache*, int slot);
@@ -43,7 +44,8 @@ int blm_cache_length(const BlmCache*, int slot);         // -1 if the slot is no
 // Pages for n sequences that grow by n_new[i] tokens each: all of them or none.  On
 // BLM_E_OVERFLOW detail[0] is the length asked for and detail[1] the maximum.
 int blm_cache_reserve(BlmCache*, int n, const int* slots, const int* n_new, int* detail);
-// The reserved step has run: the sequence is n longer; pages that fell out of a window go back.
+// The reserved step has run: the sequence is n longer; pages that fell out of a window and hold none of the
+// first keys to keep go back.
 int blm_cache_advance(BlmCache*, int slot, int n);
 // the same for the n sequences of a step, each by counts[i]: checked for all of them first
 int blm_cache_advance_all(BlmCache*, int n, const int* slots, const int* counts);

@@ -10,7 +10,7 @@ import torch
 
 from . import build as _build
 
-ABI_VERSION = 38
+ABI_VERSION = 39
 _lib = None
 _lock = threading.Lock()
 
@@ -45,7 +45,7 @@ _SIGNATURES = {
                              _c_int, _c_int, _c_int, _c_void_p],
     "blm_qkv_prepare": [_c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int,
                         _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                        _c_void_p, _c_void_p],
+                        _c_void_p, _c_int, _c_float, _c_void_p],
     "blm_sigmoid_gate": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "blm_gelu_glu": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
     "blm_softcap": [_c_void_p, ctypes.c_longlong, _c_float, _c_void_p],
@@ -54,15 +54,31 @@ _SIGNATURES = {
                               _c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_float, _c_int, _c_void_p],
     "blm_scaled_add": [_c_void_p, _c_int, _c_int, _c_int] + [_c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_int] * 4
                       + [_c_void_p],
-    "blm_moe_route_grouped": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int,
-                              _c_void_p],
+    "blm_moe_route_grouped": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p,
+                              _c_int, _c_void_p],
+    "blm_moe_gate_clamped": [_c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float,
+                             _c_void_p],
+    "blm_relu2": [_c_void_p, _c_void_p, _c_int, ctypes.c_longlong, _c_void_p],
+    "blm_post_norm": [_c_void_p] + [_c_void_p, _c_int, _c_int, ctypes.c_longlong, _c_float, _c_void_p, _c_float] * 2
+                     + [_c_void_p, _c_float, _c_int, _c_void_p, _c_int, _c_void_p, _c_float, _c_void_p, _c_int, _c_int, _c_void_p,
+                        _c_int, _c_int, _c_void_p],
+    "blm_embed_positions": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int,
+                            _c_int, _c_int, _c_int, _c_int, _c_void_p],
+    "blm_mm_step": [_c_void_p, _c_int, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_float, _c_float, _c_void_p, _c_float,
+                    _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int,
+                    _c_int, _c_int, _c_void_p, _c_void_p],
+    "blm_mm_chunks_init": [],
+    "blm_mm_chunks_supported": [_c_int, _c_int, _c_int],
+    "blm_mm_chunks": [_c_void_p, _c_int, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_float, _c_float, _c_void_p, _c_float,
+                      _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
+                      _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "blm_sink_attn_mfma_supported": [_c_int, _c_int],
     "blm_sink_attn_mfma": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                            _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                            _c_int, _c_float, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p],
     "blm_sink_attn": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                       _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int,
-                      _c_void_p],
+                      _c_int, _c_float, _c_void_p],
     "blm_streams_norm": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, ctypes.c_longlong, _c_void_p, _c_void_p, _c_void_p,
                          _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_float, _c_float,
                          _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p],
@@ -96,12 +112,12 @@ _SIGNATURES = {
                        _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p],
     "blm_attn_decode": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int,
                         _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int,
-                        _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p],
+                        _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_float, _c_void_p],
     "blm_attn_decode_supported": [_c_int, _c_int, _c_int],
     "blm_attn_prefill_mfma_supported": [_c_int, _c_int, _c_int],
     "blm_attn_prefill_mfma": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int,
                               _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
-                              _c_int, _c_int, _c_void_p, _c_void_p],
+                              _c_int, _c_int, _c_void_p, _c_int, _c_float, _c_void_p],
     "blm_gemm_tiled": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int,
                        _c_int, _c_int, _c_void_p],
     "blm_gemv_skinny": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int,
@@ -409,11 +425,12 @@ def attn_prefill_queries(n_seqs, max_new, nh, nkv, hd, compute_units):
 
 
 def attn_prefill_mfma(q, q_row_stride, out, positions, cu_seqlens, block_table, kcache, vcache, page_size,
-                      n_seqs, max_new, nh, nkv, hd, scale, window=0, queries=16, sinks=None):
+                      n_seqs, max_new, nh, nkv, hd, scale, window=0, queries=16, sinks=None, keep_first=0, softcap=0.0):
     """Causal attention of packed sequences over their cached keys on the matrix cores (bfloat16).
     Rows cu_seqlens[b] .. cu_seqlens[b+1] of q and out belong to sequence b; max_new is the most
     rows any sequence has.  queries: 16 or 32 query rows per wavefront (attn_prefill_queries chooses).
-    sinks (float32 [heads]): the softmax's denominator also holds exp(sinks[h]), a logit without key or value."""
+    sinks (float32 [heads]): the softmax's denominator also holds exp(sinks[h]), a logit without key or value.
+    keep_first: a sequence's first keys that stay visible before the window; softcap c > 0: scores s <- c tanh(s / c)."""
     _gpu(q, out, positions, cu_seqlens, block_table, kcache, vcache, sinks)
     if sinks is not None:
         _f32("sinks", sinks, nh)
@@ -429,14 +446,15 @@ def attn_prefill_mfma(q, q_row_stride, out, positions, cu_seqlens, block_table, 
         raise KernelError("attn_prefill_mfma: the page table has fewer rows than there are sequences")
     _call("blm_attn_prefill_mfma", q.data_ptr(), q_row_stride, out.data_ptr(), _code(out), positions.data_ptr(),
           cu_seqlens.data_ptr(), block_table.data_ptr(), block_table.shape[1], kcache.data_ptr(), vcache.data_ptr(),
-          page_size, int(n_seqs), int(max_new), nh, nkv, hd, float(scale), int(window), int(queries), _ptr(sinks), _stream())
+          page_size, int(n_seqs), int(max_new), nh, nkv, hd, float(scale), int(window), int(queries), _ptr(sinks),
+          int(keep_first), float(softcap), _stream())
     return out
 
 
 def attn_decode(q, q_row_stride, out, positions, token_seq, block_table, kcache, vcache, page_size,
-                nh, nkv, hd, scale, window=0, n_splits=1, sinks=None):
-    """Attention for few query tokens over long key ranges, the key range cut into n_splits.  sinks: as for
-    attn_prefill_mfma."""
+                nh, nkv, hd, scale, window=0, n_splits=1, sinks=None, keep_first=0, softcap=0.0):
+    """Attention for few query tokens over long key ranges, the key range cut into n_splits.  sinks, keep_first,
+    softcap: as for attn_prefill_mfma."""
     _gpu(q, out, positions, token_seq, block_table, kcache, vcache, sinks)
     if sinks is not None:
         _f32("sinks", sinks, nh)
@@ -457,7 +475,7 @@ def attn_decode(q, q_row_stride, out, positions, token_seq, block_table, kcache,
     _call("blm_attn_decode", q.data_ptr(), q_row_stride, out.data_ptr(), _code(out), positions.data_ptr(),
           token_seq.data_ptr(), block_table.data_ptr(), block_table.shape[1], kcache.data_ptr(), vcache.data_ptr(),
           page_size, T, nh, nkv, hd, float(scale), int(window), n_splits, _ptr(part_o), _ptr(part_ml),
-          _ptr(arrivals), _ptr(sinks), _stream())
+          _ptr(arrivals), _ptr(sinks), int(keep_first), float(softcap), _stream())
     return out
 
 
@@ -1268,12 +1286,16 @@ def moe_gate(gate_up, weights, out, n_experts, expert_inner):
     return out
 
 
-def moe_route_grouped(logits, correction, n_experts, n_identity, groups, keep, top, weights):
+def moe_route_grouped(logits, correction, n_experts, n_identity, groups, keep, top, weights, score="softmax", renormalize=True):
     """weights [T, E + 1] float32 from logits [T, >= E + n_identity] float32: scores are the softmax over all E + n_identity
     logits; the choice goes by score + correction (None: the score) among the experts of the `keep` best of `groups`
     equal groups of neighbours (a group's rank: its largest choice; groups <= 1: among all); the `top` chosen experts'
     weights are their scores over the sum of the chosen scores.  Column e < E: expert e's weight or zero; column E: the
-    weights of the chosen ones among the last n_identity (experts that pass their input through), added up."""
+    weights of the chosen ones among the last n_identity (experts that pass their input through), added up.
+    score "sigmoid": an expert's score is the sigmoid of its logit; renormalize False: the weights are the chosen scores
+    as they are."""
+    if score not in ("softmax", "sigmoid"):
+        raise KernelError(f"moe_route_grouped: score {score!r} unknown (softmax, sigmoid)")
     _gpu(logits, correction, weights)
     T = logits.shape[0]
     _f32("logits", logits); _f32("weights", weights, T * (n_experts + 1))
@@ -1282,8 +1304,165 @@ def moe_route_grouped(logits, correction, n_experts, n_identity, groups, keep, t
     if logits.dim() != 2 or tuple(weights.shape) != (T, n_experts + 1):
         raise KernelError("moe_route_grouped: logits [T, N], weights [T, E + 1]")
     _call("blm_moe_route_grouped", logits.data_ptr(), logits.shape[1], _ptr(correction), int(n_experts), int(n_identity),
-          int(groups), int(keep), int(top), weights.data_ptr(), T, _stream())
+          int(groups), int(keep), int(top), 1 if score == "sigmoid" else 0, 1 if renormalize else 0, weights.data_ptr(), T,
+          _stream())
     return weights
+
+
+def moe_gate_clamped(gate_up, weights, out, n_experts, expert_inner, limit, alpha, shared_limit=None):
+    """out [T, I] from gate_up [T, 2 I] (gate columns, then up columns): column i of expert e = i // expert_inner is
+    g * sigmoid(alpha g) * (u + 1) with g = min(w gate, limit), u = clamp(w up, -limit, limit) and w = weights[t, e], the
+    token's share on the expert's input; zero where w is zero.  Columns from n_experts * expert_inner on belong to a
+    shared expert: w = 1 and shared_limit."""
+    _gpu(gate_up, weights, out)
+    _contig("gate_up", gate_up); _contig("out", out)
+    T, I = out.shape
+    _f32("weights", weights, T * (n_experts + 1))
+    if tuple(gate_up.shape) != (T, 2 * I) or gate_up.dtype != out.dtype or I < n_experts * expert_inner:
+        raise KernelError(f"moe_gate_clamped: gate_up {tuple(gate_up.shape)} and out {tuple(out.shape)} do not fit")
+    if I > n_experts * expert_inner and shared_limit is None:
+        raise KernelError("moe_gate_clamped: the shared expert's columns need their limit")
+    _call("blm_moe_gate_clamped", gate_up.data_ptr(), weights.data_ptr(), out.data_ptr(), _code(out), T, I, int(n_experts),
+          int(expert_inner), float(limit), float(shared_limit or 0.0), float(alpha), _stream())
+    return out
+
+
+def relu2(z, out):
+    """max(z, 0)^2, element by element (out may be z)."""
+    _gpu(z, out)
+    _contig("z", z); _contig("out", out)
+    if z.shape != out.shape or z.dtype != out.dtype:
+        raise KernelError("relu2: input and output must agree in shape and dtype")
+    _call("blm_relu2", z.data_ptr(), out.data_ptr(), _code(z), z.numel(), _stream())
+    return out
+
+
+MAX_NORMED_TERMS = 2
+
+
+def post_norm(h, terms, post=None, fresh=False, vec=None, write_h=True, gamma=None, eps=0.0, out=None, rows=None):
+    """Sublayer results that are normed before they join the float32 residual h [T, D], the join, and what follows it:
+        y = sum_i scale_i * (n(y_i, eps_i) * gamma_i, or y_i where gamma_i is None)
+        y = n(y, post_eps) * post_gamma               if post = (post_gamma, post_eps)
+        v = (0 if fresh else h[r]) + vec + y;  h[r] = v if write_h
+        out[i] = n(v, eps) * gamma, or v where gamma is None            (out None: the residual alone)
+    with n(x, eps) = x / sqrt(mean(x^2) + eps) and r = rows[i] if rows is given, else i.  terms: up to two of
+    (y, scale, gamma, eps), y [T, D] in a kernel dtype or float32 planes [P, T, D] that are summed.  Weights and vec are
+    float32 [D].  out [n, D] may be a view of wider rows."""
+    _gpu(h, vec, gamma, out, rows)
+    if h.dtype != torch.float32 or h.dim() != 2:
+        raise KernelError("post_norm: the residual stream must be float32 [T, D]")
+    _contig("h", h)
+    T, D = h.shape
+    if not 1 <= len(terms) <= MAX_NORMED_TERMS:
+        raise KernelError(f"post_norm: {len(terms)} results (1 to {MAX_NORMED_TERMS})")
+    args = []
+    for y, scale, g, e in terms:
+        _gpu(y, g)
+        planes, code = _planes("post_norm", y, T, D)
+        if g is not None:
+            _f32("gamma of a result", g, D)
+        args += [y.data_ptr(), code, planes, T * D, float(scale), _ptr(g), float(e)]
+    if len(terms) == 1:
+        args += [0, 0, 1, 0, 0.0, 0, 0.0]
+    if post is not None:
+        _gpu(post[0]); _f32("post gamma", post[0], D)
+    for name, v in (("vec", vec), ("gamma", gamma)):
+        if v is not None:
+            _f32(name, v, D)
+    n = T if rows is None else rows.shape[0]
+    if rows is not None:
+        _i32("rows", rows, n)
+        if write_h:
+            raise KernelError("post_norm: listed rows are read, not written")
+    if out is not None and (tuple(out.shape) != (n, D) or out.stride(1) != 1 or out.dtype not in DTYPE_CODE):
+        raise KernelError(f"post_norm: out {tuple(out.shape)} must be [{n}, {D}] with unit stride along its rows")
+    _call("blm_post_norm", h.data_ptr(), *args, _ptr(post[0]) if post else 0, float(post[1]) if post else 0.0, 1 if fresh else 0,
+          _ptr(vec), 1 if write_h else 0, _ptr(gamma), float(eps), _ptr(out), _code(out) if out is not None else 0,
+          out.stride(0) if out is not None else 0, _ptr(rows), n, D, _stream())
+    return out
+
+
+def embed_positions(table, ids, positions, turns, out_h, copy=None, source=None):
+    """out_h[t] = table[id_t] as float32, plus (turns float64 [ceil(D / 2)], or None) at entries 2i and 2i + 1 the sine and
+    cosine of positions[t] * turns[i] full turns.  source = (rows, cell): as for embed_gather_from.  copy [T, D] (may be
+    a view of wider rows): the rows once more in its dtype."""
+    _gpu(table, ids, positions, turns, out_h, copy)
+    T, D, copies = _embed_shape("embed_positions", table, out_h)
+    if copies != 1:
+        raise KernelError("embed_positions: one residual stream")
+    _i32("ids", ids, T); _i32("positions", positions, T)
+    _contig("table", table); _contig("h", out_h)
+    if turns is not None and (turns.dtype != torch.float64 or turns.numel() != (D + 1) // 2 or not turns.is_contiguous()):
+        raise KernelError(f"embed_positions: turns must be float64 [{(D + 1) // 2}]")
+    if copy is not None and (tuple(copy.shape) != (T, D) or copy.stride(1) != 1):
+        raise KernelError("embed_positions: the copy is [T, D] with unit stride along its rows")
+    rows = cell = None
+    if source is not None:
+        rows, cell = source
+        _gpu(rows, cell); _i32("source_rows", rows, T)
+        if cell.dtype != torch.int64 or cell.numel() != 1:
+            raise KernelError("embed_positions: the cell is one int64 on the device")
+    _call("blm_embed_positions", table.data_ptr(), _code(table), ids.data_ptr(), _ptr(rows), _ptr(cell), positions.data_ptr(),
+          _ptr(turns), out_h.data_ptr(), _ptr(copy), _code(copy) if copy is not None else 0,
+          copy.stride(0) if copy is not None else 0, T, D, table.shape[0], _stream())
+    return out_h
+
+
+_mm_ready = set()
+
+
+def matrix_memory_init(device=None):
+    """Once per device, outside any stream capture, before the first matrix_memory of a prompt (its kernels take more
+    shared memory than a kernel gets without asking)."""
+    index = torch.device(device or "cuda").index
+    index = torch.cuda.current_device() if index is None else index
+    if index not in _mm_ready:
+        with torch.cuda.device(index):
+            _call("blm_mm_chunks_init")
+        _mm_ready.add(index)
+
+
+def matrix_memory_chunks_supported(dk, dv, dtype):
+    return dtype in DTYPE_CODE and bool(library().blm_mm_chunks_supported(int(dk), int(dv), DTYPE_CODE[dtype]))
+
+
+def matrix_memory(proj, logits, bias_i, bias_f, cap, q_scale, norm_w, eps, state, out, step, H, dk, dv, chunks):
+    """The stabilised matrix memory (csrc/matrix_memory.hip) over proj [T, >= 2 H dk + 2 H dv] (queries, keys, values,
+    output-gate logits) with gate logits float32 [T, >= 2 H] (input gates, forget gates; before their biases and the
+    cap), then every head's norm with norm_w [H * dv] and the sigmoid of the output gate's logits.  state = (S [slots,
+    H, dk, dv], n [slots, H, dk], m [slots, H]) float32, read and left updated.  out [T, H * dv].  chunks: the form for
+    prompts (proj in out's dtype); else the form for steps of few tokens per sequence (proj may be float32)."""
+    S, n_state, m_state = state
+    _gpu(proj, logits, bias_i, bias_f, norm_w, S, n_state, m_state, out)
+    T = proj.shape[0]
+    _f32("bias_i", bias_i, H); _f32("bias_f", bias_f, H); _f32("norm_w", norm_w, H * dv)
+    _f32("S", S); _f32("n", n_state); _f32("m", m_state)
+    _contig("out", out)
+    if logits.dtype != torch.float32 or logits.dim() != 2 or logits.shape[0] != T or logits.shape[1] < 2 * H or logits.stride(1) != 1:
+        raise KernelError("matrix_memory: gate logits must be float32 [T, >= 2 H]")
+    if proj.stride(1) != 1 or tuple(out.shape) != (T, H * dv) or tuple(S.shape[1:]) != (H, dk, dv) or T != step.n_tokens             or tuple(n_state.shape[1:]) != (H, dk) or tuple(m_state.shape[1:]) != (H,) or proj.shape[1] < 2 * H * (dk + dv):
+        raise KernelError("matrix_memory: shapes do not fit")
+    if proj.dtype != out.dtype and (chunks or proj.dtype != torch.float32):
+        raise KernelError("matrix_memory: the projection must be of out's dtype (or float32 in steps of few tokens)")
+    B = step.n_seqs
+    o_raw = torch.empty(T, H * dv, dtype=torch.float32, device=proj.device)
+    head = (proj.data_ptr(), _code(proj), proj.stride(0), logits.data_ptr(), logits.stride(0), bias_i.data_ptr(), bias_f.data_ptr(),
+            float(cap), float(q_scale), norm_w.data_ptr(), float(eps), S.data_ptr(), n_state.data_ptr(), m_state.data_ptr())
+    if not chunks:
+        counters = arrival_counters(out.device)
+        if B * H > counters.numel():
+            raise KernelError(f"matrix_memory: {B} sequences of {H} heads are more than there are arrival counters")
+        _call("blm_mm_step", *head, o_raw.data_ptr(), out.data_ptr(), _code(out), step.cu_seqlens.data_ptr(),
+              step.seq_slots.data_ptr(), T, B, H, dk, dv, counters.data_ptr(), _stream())
+        return out
+    n_seg = -(-step.max_new // LIGHTNING_CHUNK)
+    f32 = lambda *shape: torch.empty(*shape, dtype=torch.float32, device=proj.device)
+    gates, chunk, seg, seg_n = f32(3, H, T), f32(B, n_seg, H, 2), f32(B, n_seg, H, dk, dv), f32(B, n_seg, H, dk)
+    _call("blm_mm_chunks", *head, gates.data_ptr(), chunk.data_ptr(), seg.data_ptr(), seg_n.data_ptr(), o_raw.data_ptr(),
+          out.data_ptr(), step.cu_seqlens.data_ptr(), step.seq_slots.data_ptr(), step.token_seq.data_ptr(), T, B, H, dk, dv,
+          step.max_new, n_seg, _stream())
+    return out
 
 
 MAX_ADD_TERMS = 4
@@ -1431,13 +1610,14 @@ def lightning_chunks(proj, powers, norm_w, eps, state, o_raw, out, step, H, dk, 
 
 
 def qkv_prepare(qkv, bias, cos_sin, rot, step, block_table, kcache, vcache, page_size, H, G, dk, dv, write_kv=True,
-                adjacent=False, values_are_keys=False, q_scale=None):
+                adjacent=False, values_are_keys=False, q_scale=None, unit_norm_eps=None):
     """Bias, rotation of the first `rot` lanes of every query and key head by the token's position (lane i with
     lane i + rot/2, or with adjacent lanes 2i and 2i + 1; cos_sin float32 [positions, >= rot/2, 2] rows of exactly
     rot/2 pairs), queries in place, rotated keys and values into the pages (key pages [pages, G, page, dk], value pages
     [pages, G, dv, page]).  write_kv False: qkv holds queries only and nothing is stored.  values_are_keys: the rows
     hold no values; a token's values are its keys as projected, before the rotation (dv = dk).  q_scale (float32 [H]
-    or None): query head h is multiplied by q_scale[h] behind the rotation."""
+    or None): query head h is multiplied by q_scale[h] behind the rotation.  unit_norm_eps (a number or None): every
+    query and key head, with its bias, is divided by sqrt(mean of its squares + unit_norm_eps) in front of the rotation."""
     _gpu(qkv, bias, cos_sin, block_table, kcache, vcache, q_scale)
     if q_scale is not None:
         _f32("q_scale", q_scale, H)
@@ -1464,14 +1644,16 @@ def qkv_prepare(qkv, bias, cos_sin, rot, step, block_table, kcache, vcache, page
           step.positions.data_ptr(), step.token_seq.data_ptr(), _ptr(block_table) if write_kv else 0,
           block_table.shape[1] if write_kv else 0, _ptr(kcache) if write_kv else 0, _ptr(vcache) if write_kv else 0,
           page_size, T, H, G, dk, dv, 1 if write_kv else 0, 1 if adjacent else 0, 1 if values_are_keys else 0, _ptr(q_scale),
-          _stream())
+          0 if unit_norm_eps is None else 1, float(unit_norm_eps or 0.0), _stream())
     return qkv
 
 
-def sink_attn(q, out, sinks, mix, step, block_table, kcache, vcache, page_size, H, G, dk, dv, scale, window):
+def sink_attn(q, out, sinks, mix, step, block_table, kcache, vcache, page_size, H, G, dk, dv, scale, window, keep_first=0,
+              softcap=0.0):
     """Attention whose softmax denominator also holds exp(sinks[h]) (sinks None: a plain softmax) and whose weights
     are mixed between heads by mix [H, H] (None: not mixed) before head h reads the values of its own key-value head.
-    q [T, >= H dk] rows (queries already rotated), out [T, H * dv] in q's dtype."""
+    q [T, >= H dk] rows (queries already rotated), out [T, H * dv] in q's dtype.  keep_first: a sequence's first keys
+    that stay visible before the window; softcap c > 0: scores s <- c tanh(s / c)."""
     _gpu(q, out, sinks, mix, block_table, kcache, vcache)
     T = q.shape[0]
     _contig("out", out); _contig("kcache", kcache); _contig("vcache", vcache); _i32("block_table", block_table)
@@ -1487,7 +1669,8 @@ def sink_attn(q, out, sinks, mix, step, block_table, kcache, vcache, page_size, 
     A = torch.empty(T, H, G if mix is not None else 1, dv, dtype=torch.float32, device=q.device)
     _call("blm_sink_attn", q.data_ptr(), q.stride(0), out.data_ptr(), _code(q), A.data_ptr(), _ptr(sinks), _ptr(mix),
           step.positions.data_ptr(), step.token_seq.data_ptr(), block_table.data_ptr(), block_table.shape[1],
-          kcache.data_ptr(), vcache.data_ptr(), page_size, T, H, G, dk, dv, float(scale), int(window), _stream())
+          kcache.data_ptr(), vcache.data_ptr(), page_size, T, H, G, dk, dv, float(scale), int(window), int(keep_first),
+          float(softcap), _stream())
     return out
 
 

@@ -506,6 +506,116 @@ extern "C" int blm_moe_gate(const void* gate_up, const float* weights, void* out
   return 0;
 }
 
+// The same for clamped gated experts whose weight is on their input: with w the token's weight for the column's expert,
+// g = min(w gate, limit), u = clamp(w up, -limit, limit), out = g * sigmoid(alpha g) * (u + 1), zero where w is zero.
+// The columns from E * ffe on are a shared expert's: w = 1 and a limit of its own.
+__device__ __forceinline__ float pb_clamped(float g, float u, float limit, float alpha) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * pb_sigmoid(alpha * g) * (u + 1.0f);
+}
+template <typename TA>
+__global__ void moe_gate_clamped_kernel(const TA* __restrict__ gate_up, const float* __restrict__ weights, TA* __restrict__ out,
+                                        long long n, int I, int E, int ffe, float limit, float shared_limit, float alpha) {
+  const long long stride = (long long)gridDim.x * blockDim.x;
+  for (long long e = (long long)blockIdx.x * blockDim.x + threadIdx.x; e < n; e += stride) {
+    const long long t = e / I;
+    const int i = (int)(e - t * I);
+    const bool shared = i >= E * ffe;
+    const float w = shared ? 1.0f : weights[(size_t)t * (E + 1) + i / ffe];
+    float v = 0.f;
+    if (w != 0.f)
+      v = pb_clamped(w * to_float(gate_up[(size_t)t * 2 * I + i]), w * to_float(gate_up[(size_t)t * 2 * I + I + i]),
+                     shared ? shared_limit : limit, alpha);
+    out[e] = from_float<TA>(v);
+  }
+}
+// eight bfloat16 at a time (the experts' inner sizes and I multiples of 8: eight neighbours belong to one expert)
+__global__ void moe_gate_clamped8_kernel(const bf16* __restrict__ gate_up, const float* __restrict__ weights, bf16* __restrict__ out,
+                                         long long n8, int I8, int E, int ffe8, float limit, float shared_limit, float alpha) {
+  const long long stride = (long long)gridDim.x * blockDim.x;
+  for (long long e = (long long)blockIdx.x * blockDim.x + threadIdx.x; e < n8; e += stride) {
+    const long long t = e / I8;
+    const int i = (int)(e - t * I8);
+    const bool shared = i >= E * ffe8;
+    const float w = shared ? 1.0f : weights[(size_t)t * (E + 1) + i / ffe8];
+    const float lim = shared ? shared_limit : limit;
+    uint32_t r[4] = {0u, 0u, 0u, 0u};
+    if (w != 0.f) {
+      const uint4 g4 = *reinterpret_cast<const uint4*>(gate_up + ((size_t)t * 2 * I8 + i) * 8);
+      const uint4 u4 = *reinterpret_cast<const uint4*>(gate_up + ((size_t)t * 2 * I8 + I8 + i) * 8);
+      const uint32_t gw[4] = {g4.x, g4.y, g4.z, g4.w}, uw[4] = {u4.x, u4.y, u4.z, u4.w};
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+        r[k] = f32x2_to_bf16x2_bits(pb_clamped(w * pb_lo(gw[k]), w * pb_lo(uw[k]), lim, alpha),
+                                    pb_clamped(w * pb_hi(gw[k]), w * pb_hi(uw[k]), lim, alpha));
+    }
+    *reinterpret_cast<uint4*>(out + (size_t)e * 8) = make_uint4(r[0], r[1], r[2], r[3]);
+  }
+}
+
+extern "C" int blm_moe_gate_clamped(const void* gate_up, const float* weights, void* out, int dtype, int T, int I, int E, int ffe,
+                                    float limit, float shared_limit, float alpha, hipStream_t stream) {
+  BLM_REQUIRE(T > 0 && E > 0 && ffe > 0 && I >= E * ffe && limit > 0.f && (I == E * ffe || shared_limit > 0.f),
+              "moe_gate_clamped: bad sizes T=%d I=%d experts=%d of %d, limits %g and %g", T, I, E, ffe, (double)limit, (double)shared_limit);
+  const long long n = (long long)T * I;
+  const unsigned blocks = (unsigned)((n + 255) / 256 < 65535 ? (n + 255) / 256 : 65535);
+  if (dtype == BLM_F32)
+    hipLaunchKernelGGL(moe_gate_clamped_kernel<float>, dim3(blocks), dim3(256), 0, stream, (const float*)gate_up, weights, (float*)out, n, I,
+                       E, ffe, limit, shared_limit, alpha);
+  else if (dtype == BLM_BF16 && I % 8 == 0 && ffe % 8 == 0 && ((size_t)gate_up & 15) == 0 && ((size_t)out & 15) == 0) {
+    const long long n8 = n / 8;
+    const unsigned b8 = (unsigned)((n8 + 255) / 256 < 65535 ? (n8 + 255) / 256 : 65535);
+    hipLaunchKernelGGL(moe_gate_clamped8_kernel, dim3(b8), dim3(256), 0, stream, (const bf16*)gate_up, weights, (bf16*)out, n8, I / 8, E,
+                       ffe / 8, limit, shared_limit, alpha);
+  } else if (dtype == BLM_BF16)
+    hipLaunchKernelGGL(moe_gate_clamped_kernel<bf16>, dim3(blocks), dim3(256), 0, stream, (const bf16*)gate_up, weights, (bf16*)out, n, I, E,
+                       ffe, limit, shared_limit, alpha);
+  else
+    return blm_fail("moe_gate_clamped: unsupported dtype %d", dtype);
+  BLM_LAUNCH_CHECK("moe_gate_clamped");
+  return 0;
+}
+
+// ---------------------------------------------------------------------------------------
+// Squared ReLU, element by element: out = max(z, 0)^2 (out may be z itself).
+// ---------------------------------------------------------------------------------------
+template <typename TA>
+__global__ void relu2_kernel(const TA* z, TA* out, long long n) {
+  const long long stride = (long long)gridDim.x * blockDim.x;
+  for (long long e = (long long)blockIdx.x * blockDim.x + threadIdx.x; e < n; e += stride) {
+    const float v = fmaxf(to_float(z[e]), 0.f);
+    out[e] = from_float<TA>(v * v);
+  }
+}
+__global__ void relu2_8_kernel(const bf16* z, bf16* out, long long n8) {
+  const long long stride = (long long)gridDim.x * blockDim.x;
+  for (long long e = (long long)blockIdx.x * blockDim.x + threadIdx.x; e < n8; e += stride) {
+    const uint4 v = reinterpret_cast<const uint4*>(z)[e];
+    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+    uint32_t r[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const float a = fmaxf(pb_lo(w[k]), 0.f), b = fmaxf(pb_hi(w[k]), 0.f);
+      r[k] = f32x2_to_bf16x2_bits(a * a, b * b);
+    }
+    reinterpret_cast<uint4*>(out)[e] = make_uint4(r[0], r[1], r[2], r[3]);
+  }
+}
+extern "C" int blm_relu2(const void* z, void* out, int dtype, long long n, hipStream_t stream) {
+  BLM_REQUIRE(n > 0, "relu2: nothing to do");
+  const unsigned blocks = (unsigned)((n + 255) / 256 < 65535 ? (n + 255) / 256 : 65535);
+  if (dtype == BLM_F32) hipLaunchKernelGGL(relu2_kernel<float>, dim3(blocks), dim3(256), 0, stream, (const float*)z, (float*)out, n);
+  else if (dtype == BLM_BF16 && n % 8 == 0 && (((size_t)z | (size_t)out) & 15) == 0) {
+    const long long n8 = n / 8;
+    const unsigned b8 = (unsigned)((n8 + 255) / 256 < 65535 ? (n8 + 255) / 256 : 65535);
+    hipLaunchKernelGGL(relu2_8_kernel, dim3(b8), dim3(256), 0, stream, (const bf16*)z, (bf16*)out, n8);
+  } else if (dtype == BLM_BF16) hipLaunchKernelGGL(relu2_kernel<bf16>, dim3(blocks), dim3(256), 0, stream, (const bf16*)z, (bf16*)out, n);
+  else return blm_fail("relu2: unsupported dtype %d", dtype);
+  BLM_LAUNCH_CHECK("relu2");
+  return 0;
+}
+
 // ---------------------------------------------------------------------------------------
 // Several sublayers' results into the residual at once, each with a coefficient per channel and (optionally) per
 // token:  h[t][c] += sum_i chan_i[c] * row_i[t] * sum_p y_i[p][t][c]  in float.  A term's y is [T][D] in any kernel
@@ -636,8 +746,9 @@ extern "C" int blm_scaled_add(float* h, int T, int D, int n_terms,
 // choice = s + correction (null: none).  The N experts form `groups` equal groups of neighbours; a group's score is its
 // largest choice; only experts of the `keep` best groups can be chosen (groups <= 1: all can).  The `top` largest
 // choices are taken (the lower index wins a tie); their weights are s (without the correction) over the sum of the
-// chosen s (+ 1e-20).  weights [T][E + 1] float: a real expert's weight or 0, and at E the sum of the weights of the
-// chosen pass-through experts.
+// chosen s (+ 1e-20), or (renorm 0) the chosen s as they are.  sigmoid 1: s = sigmoid(logits), each on its own.
+// weights [T][E + 1] float: a real expert's weight or 0, and at E the sum of the weights of the chosen pass-through
+// experts.
 // ---------------------------------------------------------------------------------------
 #define PB_MAX_ROUTED 256
 #define PB_ROUTED_PER_LANE (PB_MAX_ROUTED / BLM_WAVE)
@@ -657,7 +768,8 @@ __device__ __forceinline__ void pb_wave_best(float& v, int& i) {
 // groups' ranks and the kept groups pass through the wavefront's piece of shared memory.
 __global__ void __launch_bounds__(256)
     moe_route_grouped_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ correction, int E,
-                             int n_identity, int groups, int keep, int top, float* __restrict__ weights, int T) {
+                             int n_identity, int groups, int keep, int top, int sigmoid, int renorm,
+                             float* __restrict__ weights, int T) {
   __shared__ float sm_choice[4][PB_MAX_ROUTED];
   __shared__ int sm_kept[4][PB_MAX_ROUTED];
   const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
@@ -678,10 +790,11 @@ __global__ void __launch_bounds__(256)
   float denom = 0.f;
 #pragma unroll
   for (int k = 0; k < PB_ROUTED_PER_LANE; ++k) {
-    score[k] = lane + k * BLM_WAVE < N ? expf(zs[k] - largest) : 0.f;
+    const bool real = lane + k * BLM_WAVE < N;
+    score[k] = !real ? 0.f : sigmoid ? 1.0f / (1.0f + expf(-zs[k])) : expf(zs[k] - largest);
     denom += score[k];
   }
-  const float inv = 1.0f / wave_sum(denom);
+  const float inv = sigmoid ? 1.0f : 1.0f / wave_sum(denom);
 #pragma unroll
   for (int k = 0; k < PB_ROUTED_PER_LANE; ++k) {
     const int e = lane + k * BLM_WAVE;
@@ -745,7 +858,7 @@ __global__ void __launch_bounds__(256)
       if (lane + k * BLM_WAVE == bi) { mine[k] = true; open[k] = false; sum += score[k]; }
   }
   sum = wave_sum(sum);
-  const float norm = 1.0f / (sum + 1e-20f);
+  const float norm = renorm ? 1.0f / (sum + 1e-20f) : 1.0f;
   // real experts' weights straight out; the pass-through experts' added up over the wavefront
   float passed = 0.f;
 #pragma unroll
@@ -759,7 +872,7 @@ __global__ void __launch_bounds__(256)
 }
 
 extern "C" int blm_moe_route_grouped(const float* logits, int ld, const float* correction, int E, int n_identity, int groups,
-                                     int keep, int top, float* weights, int T, hipStream_t stream) {
+                                     int keep, int top, int sigmoid, int renorm, float* weights, int T, hipStream_t stream) {
   const int N = E + n_identity;
   BLM_REQUIRE(T > 0 && E >= 0 && n_identity >= 0 && N >= 1 && N <= PB_MAX_ROUTED && ld >= N && top >= 1 && top <= N,
               "moe_route_grouped: bad sizes T=%d experts=%d+%d (at most %d) top=%d", T, E, n_identity, PB_MAX_ROUTED, top);
@@ -767,7 +880,7 @@ extern "C" int blm_moe_route_grouped(const float* logits, int ld, const float* c
               N, groups, keep);
   BLM_REQUIRE(top <= (groups > 1 ? keep * (N / groups) : N), "moe_route_grouped: top=%d is more than the kept groups hold", top);
   hipLaunchKernelGGL(moe_route_grouped_kernel, dim3((T + 3) / 4), dim3(256), 0, stream, logits, ld, correction, E,
-                     n_identity, groups, keep, top, weights, T);
+                     n_identity, groups, keep, top, sigmoid, renorm, weights, T);
   BLM_LAUNCH_CHECK("moe_route_grouped");
   return 0;
 }

@@ -12,11 +12,7 @@
 // decoding; gated linear attention also cuts a prompt into segments that several wavefronts walk at once.
 //
 // Also here: the short causal convolution in front of the delta rule with its per-sequence history.
-#include "common.h"
-
-__device__ __forceinline__ float blm_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float blm_silu(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float blm_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+#include "chunk_form.h"
 
 // Two shapes of a wavefront (LPC lanes per column, 64 / LPC columns; lane group g holds rows g * ROWS .. + ROWS - 1):
 // 4 lanes per column for steps of few tokens per sequence (decoding): 16 neighbouring columns make the state's
@@ -177,12 +173,18 @@ __global__ void __launch_bounds__(SCAN_WAVES* BLM_WAVE)
 // Rows of padding tokens hold whatever o_raw holds (the caller clears it).
 template <typename TA>
 __global__ void __launch_bounds__(SCAN_WAVES* BLM_WAVE)
-    head_norm_kernel(const float* __restrict__ o_raw, const float* __restrict__ norm_w, const TA* __restrict__ gate,
-                     int gate_ld, int gate_mode, int H, TA* __restrict__ out, long long n_items, int dv, float eps) {
+    head_norm_kernel(const float* __restrict__ o_raw, const float* __restrict__ norm_w, int w_heads, const TA* __restrict__ gate,
+                     int gate_ld, int gate_mode, int H, TA* __restrict__ out, long long n_items, int dv, float eps,
+                     const int* __restrict__ token_seq) {
   const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
   const long long item = (long long)blockIdx.x * SCAN_WAVES + wave;
   if (item >= n_items) return;
   const float* src = o_raw + (size_t)item * dv;
+  if (token_seq && token_seq[item / H] < 0) {
+    for (int j = lane; j < dv; j += BLM_WAVE) out[(size_t)item * dv + j] = from_float<TA>(0.f);
+    return;
+  }
+  norm_w += (size_t)(item % w_heads) * dv;
   const TA* grow = gate ? gate + (size_t)(item / H) * gate_ld + (size_t)(item % H) * dv : nullptr;
   float ss = 0.f;
   for (int j = lane; j < dv; j += BLM_WAVE) ss = fmaf(src[j], src[j], ss);
@@ -202,11 +204,17 @@ __global__ void __launch_bounds__(SCAN_WAVES* BLM_WAVE)
 #define HEAD_NORM_WIDE_PER 8
 template <typename TA>
 __global__ void __launch_bounds__(256)
-    head_norm_wide_kernel(const float* __restrict__ o_raw, const float* __restrict__ norm_w, const TA* __restrict__ gate,
-                          int gate_ld, int gate_mode, int H, TA* __restrict__ out, int dv, float eps) {
+    head_norm_wide_kernel(const float* __restrict__ o_raw, const float* __restrict__ norm_w, int w_heads,
+                          const TA* __restrict__ gate, int gate_ld, int gate_mode, int H, TA* __restrict__ out, int dv, float eps,
+                          const int* __restrict__ token_seq) {
   __shared__ float part[4];
   const long long item = blockIdx.x;
   const float* src = o_raw + (size_t)item * dv;
+  if (token_seq && token_seq[item / H] < 0) {      // uniform: the whole block leaves
+    for (int j = threadIdx.x; j < dv; j += 256) out[(size_t)item * dv + j] = from_float<TA>(0.f);
+    return;
+  }
+  norm_w += (size_t)(item % w_heads) * dv;
   const TA* grow = gate ? gate + (size_t)(item / H) * gate_ld + (size_t)(item % H) * dv : nullptr;
   float x[HEAD_NORM_WIDE_PER];
   float ss = 0.f;
@@ -237,27 +245,32 @@ __global__ void __launch_bounds__(256)
   for (int j = threadIdx.x + HEAD_NORM_WIDE_PER * 256; j < dv; j += 256) put(j, src[j]);
 }
 
-static int launch_head_norm(const float* o_raw, const float* norm_w, const void* gate, int gate_ld, int gate_mode, int H,
-                            void* out, int dtype, long long items, int dv, float eps, hipStream_t stream) {
+int blm_launch_head_norm(const float* o_raw, const float* norm_w, int w_heads, const void* gate, int gate_ld, int gate_mode, int H,
+                         void* out, int dtype, long long items, int dv, float eps, const int* token_seq, hipStream_t stream) {
   if (dv >= 512 && items < (1ll << 31)) {
     if (dtype == BLM_F32)
-      hipLaunchKernelGGL(head_norm_wide_kernel<float>, dim3((unsigned)items), dim3(256), 0, stream, o_raw, norm_w,
-                         (const float*)gate, gate_ld, gate_mode, H, (float*)out, dv, eps);
+      hipLaunchKernelGGL(head_norm_wide_kernel<float>, dim3((unsigned)items), dim3(256), 0, stream, o_raw, norm_w, w_heads,
+                         (const float*)gate, gate_ld, gate_mode, H, (float*)out, dv, eps, token_seq);
     else
-      hipLaunchKernelGGL(head_norm_wide_kernel<bf16>, dim3((unsigned)items), dim3(256), 0, stream, o_raw, norm_w,
-                         (const bf16*)gate, gate_ld, gate_mode, H, (bf16*)out, dv, eps);
+      hipLaunchKernelGGL(head_norm_wide_kernel<bf16>, dim3((unsigned)items), dim3(256), 0, stream, o_raw, norm_w, w_heads,
+                         (const bf16*)gate, gate_ld, gate_mode, H, (bf16*)out, dv, eps, token_seq);
     BLM_LAUNCH_CHECK("head_norm_wide");
     return 0;
   }
   const unsigned blocks = (unsigned)((items + SCAN_WAVES - 1) / SCAN_WAVES);
   if (dtype == BLM_F32)
-    hipLaunchKernelGGL(head_norm_kernel<float>, dim3(blocks), dim3(SCAN_WAVES * BLM_WAVE), 0, stream, o_raw, norm_w,
-                       (const float*)gate, gate_ld, gate_mode, H, (float*)out, items, dv, eps);
+    hipLaunchKernelGGL(head_norm_kernel<float>, dim3(blocks), dim3(SCAN_WAVES * BLM_WAVE), 0, stream, o_raw, norm_w, w_heads,
+                       (const float*)gate, gate_ld, gate_mode, H, (float*)out, items, dv, eps, token_seq);
   else
-    hipLaunchKernelGGL(head_norm_kernel<bf16>, dim3(blocks), dim3(SCAN_WAVES * BLM_WAVE), 0, stream, o_raw, norm_w,
-                       (const bf16*)gate, gate_ld, gate_mode, H, (bf16*)out, items, dv, eps);
+    hipLaunchKernelGGL(head_norm_kernel<bf16>, dim3(blocks), dim3(SCAN_WAVES * BLM_WAVE), 0, stream, o_raw, norm_w, w_heads,
+                       (const bf16*)gate, gate_ld, gate_mode, H, (bf16*)out, items, dv, eps, token_seq);
   BLM_LAUNCH_CHECK("head_norm");
   return 0;
+}
+
+static int launch_head_norm(const float* o_raw, const float* norm_w, const void* gate, int gate_ld, int gate_mode, int H,
+                            void* out, int dtype, long long items, int dv, float eps, hipStream_t stream) {
+  return blm_launch_head_norm(o_raw, norm_w, 1, gate, gate_ld, gate_mode, H, out, dtype, items, dv, eps, nullptr, stream);
 }
 
 // Wavefronts per block and shared memory of a scan whose wavefronts each keep `vectors` per-channel vectors for a
@@ -952,17 +965,6 @@ extern "C" int blm_gla_scan(void* proj, int dtype, int ld, const void* decay_in,
 // result register r of lane l is row 8 (r / 4) + 4 (l / 32) + r % 4, column l % 32.
 // Heads of up to 128 key and 128 value channels, padded to multiples of 32 with zeros.
 // ---------------------------------------------------------------------------------------
-#define LC_CHUNK 64
-#define LC_MAX 128
-#define LC_THREADS 256
-#define LC_A_LD (LC_CHUNK + 1)
-#define LC_STEPS 8      // matrix instructions written out per turn of a loop over depth: 16 steps of depth
-#define LC_LDS_LIMIT (128 * 1024)
-typedef float lc_acc __attribute__((ext_vector_type(16)));
-
-template <typename TA>
-__device__ __forceinline__ int lc_row_pad() { return sizeof(TA) == 4 ? 1 : 2; }      // an odd number of 4-byte words per row
-
 // SiLU rounded to the rows' type.  Rows of 16 bits take the hardware's exponential and reciprocal, whose errors (about
 // 1e-6 of the result) are far below that rounding; float rows take the exact functions.
 template <typename TA>
@@ -987,66 +989,6 @@ __global__ void silu_rows_wide_kernel(TA* __restrict__ proj, int ld, int cols, l
 #pragma unroll
     for (int k = 0; k < VEC; ++k) vals[k] = lc_silu(vals[k]);
     *at = raw;
-  }
-}
-
-// A chunk's rows of one head into shared memory as they are, for N operands at once (queries, keys, values): operand p
-// is `width[p]` channels from column col0[p] on and arrives in dst[p] [64][row_ld[p]]; the tokens from n on and the channels
-// from width up to the padded width WP arrive as zeros.  Where rows and widths allow, every lane takes 16 bytes at a
-// time, has all its loads of all operands under way before it turns to the first (one trip to memory, not one per
-// operand), and leaves them as 4-byte words (row_ld and the 16-byte pieces keep every word aligned).
-template <typename TA, int N>
-struct LcOperands {
-  int col0[N], width[N], WP[N], row_ld[N];
-  TA* dst[N];
-};
-
-template <typename TA, int N>
-__device__ __forceinline__ void lc_stage(const TA* __restrict__ rows, int ld, int n, const LcOperands<TA, N>& op) {
-  constexpr int VEC = 16 / sizeof(TA);
-  bool wide = ld % VEC == 0 && (reinterpret_cast<uintptr_t>(rows) & 15) == 0;
-#pragma unroll
-  for (int p = 0; p < N; ++p) wide = wide && op.width[p] % VEC == 0 && op.col0[p] % VEC == 0 && op.width[p] <= LC_MAX;
-  if (wide) {
-    // up to 64 * 128 / VEC pieces per operand: at most 4 (16-bit rows) or 8 (float rows) per lane
-    constexpr int PER = (LC_CHUNK * LC_MAX / VEC + LC_THREADS - 1) / LC_THREADS;
-    uint4 raw[N][PER];
-    int at[N][PER];
-#pragma unroll
-    for (int p = 0; p < N; ++p) {
-      const int per_row = op.width[p] / VEC, items = LC_CHUNK * per_row;
-      const TA* src = rows + op.col0[p];
-#pragma unroll
-      for (int u = 0; u < PER; ++u) {
-        const int e = threadIdx.x + u * LC_THREADS, j = e / per_row, i = (e - j * per_row) * VEC;
-        at[p][u] = e < items ? j * op.row_ld[p] + i : -1;
-        raw[p][u] = (e < items && j < n) ? *reinterpret_cast<const uint4*>(src + (size_t)j * ld + i) : uint4{0u, 0u, 0u, 0u};
-      }
-    }
-#pragma unroll
-    for (int p = 0; p < N; ++p) {
-#pragma unroll
-      for (int u = 0; u < PER; ++u) {
-        if (at[p][u] >= 0) {
-          uint32_t* w = reinterpret_cast<uint32_t*>(op.dst[p] + at[p][u]);
-          w[0] = raw[p][u].x; w[1] = raw[p][u].y; w[2] = raw[p][u].z; w[3] = raw[p][u].w;
-        }
-      }
-      if (op.WP[p] > op.width[p]) {
-        const int extra = op.WP[p] - op.width[p];
-        for (int e = threadIdx.x; e < LC_CHUNK * extra; e += LC_THREADS)
-          op.dst[p][(e / extra) * op.row_ld[p] + op.width[p] + e % extra] = from_float<TA>(0.f);
-      }
-    }
-  } else {
-#pragma unroll
-    for (int p = 0; p < N; ++p) {
-      const TA* src = rows + op.col0[p];
-      for (int e = threadIdx.x; e < LC_CHUNK * op.WP[p]; e += LC_THREADS) {
-        const int j = e / op.WP[p], i = e - j * op.WP[p];
-        op.dst[p][j * op.row_ld[p] + i] = (j < n && i < op.width[p]) ? src[(size_t)j * ld + i] : from_float<TA>(0.f);
-      }
-    }
   }
 }
 

@@ -1,7 +1,8 @@
 // Attention over the paged cache whose softmax has a sink (one learned logit per head that takes its share of
 // the denominator and has no key and no value) and whose weights are mixed between the heads afterwards
 // ("talking heads": weight'_h(i, j) = sum_g M[h][g] weight_g(i, j), head h then reads the values of its own
-// key-value head).  Keys and values may have head sizes of their own; a window limits how far back a query sees.
+// key-value head).  Keys and values may have head sizes of their own; a window limits how far back a query sees,
+// beside which a sequence's first keep_first keys may stay visible; scores may be capped, s <- cap * tanh(s / cap).
 //
 // The mixing is linear, so it is moved behind the sum over the keys:
 //   out_h = sum_g M[h][g] * A[g][c(h)],   A[g][c] = sum_j weight_g(i, j) v_c(j),   c(h) the key-value head of h
@@ -23,6 +24,8 @@
 // lanes is (2i, 2i + 1) instead of (i, i + rot/2).  values_are_keys (dv = dk): there are no value columns; a token's
 // values are its keys as projected (with their bias), before the rotation.  q_scale [H] float or null: every lane of
 // query head h is multiplied by q_scale[h] behind the rotation (a temperature per head: the scores are linear in it).
+// unit_norm: every query and key head (with its bias) is divided by its root mean square over its lanes,
+// x / sqrt(mean(x^2) + norm_eps), in front of the rotation; values are not.  (Dynamic shared memory: one float per head.)
 // ---------------------------------------------------------------------------------------
 template <typename TA>
 __global__ void qkv_prepare_kernel(TA* __restrict__ qkv, int ld, const float* __restrict__ bias,
@@ -30,7 +33,8 @@ __global__ void qkv_prepare_kernel(TA* __restrict__ qkv, int ld, const float* __
                                    const int* __restrict__ token_seq, const int* __restrict__ block_table, int table_width,
                                    TA* __restrict__ kcache, TA* __restrict__ vcache, int page_size, int H, int G, int dk,
                                    int dv, int write_kv, int adjacent, int values_are_keys,
-                                   const float* __restrict__ q_scale) {
+                                   const float* __restrict__ q_scale, int unit_norm, float norm_eps) {
+  extern __shared__ float head_factor[];      // unit_norm: [n_rot_heads]
   const int t = blockIdx.x;
   const int b = token_seq[t];
   if (b < 0) return;
@@ -44,13 +48,27 @@ __global__ void qkv_prepare_kernel(TA* __restrict__ qkv, int ld, const float* __
     page = block_table[(size_t)b * table_width + pos / page_size];
     in_page = pos % page_size;
   }
+  if (unit_norm) {
+    const int lane = threadIdx.x & (BLM_WAVE - 1), waves = blockDim.x / BLM_WAVE;
+    for (int head = threadIdx.x / BLM_WAVE; head < n_rot_heads; head += waves) {
+      float ss = 0.f;
+      for (int d = lane; d < dk; d += BLM_WAVE) {
+        float u = to_float(row[head * dk + d]);
+        if (bias) u += bias[head * dk + d];
+        ss = fmaf(u, u, ss);
+      }
+      ss = wave_sum(ss);
+      if (lane == 0) head_factor[head] = 1.0f / sqrtf(ss / (float)dk + norm_eps);
+    }
+    __syncthreads();
+  }
   // rotating pairs and the lanes behind them, head by head (queries, then keys)
   const int per_head = half + (dk - rot);
   for (int e = threadIdx.x; e < n_rot_heads * per_head; e += blockDim.x) {
     const int head = e / per_head, i = e - head * per_head;
     const int col = head * dk;
     TA* krow = head >= H ? kcache + (((size_t)page * G + (head - H)) * page_size + in_page) * dk : nullptr;
-    const float f = (q_scale && head < H) ? q_scale[head] : 1.0f;
+    const float f = ((q_scale && head < H) ? q_scale[head] : 1.0f) * (unit_norm ? head_factor[head] : 1.0f);
     if (i < half) {
       const int la = adjacent ? 2 * i : i, lb = adjacent ? 2 * i + 1 : i + half;
       float u = to_float(row[col + la]), v = to_float(row[col + lb]);
@@ -63,7 +81,7 @@ __global__ void qkv_prepare_kernel(TA* __restrict__ qkv, int ld, const float* __
       const int lane = rot + (i - half);
       float u = to_float(row[col + lane]);
       if (bias) u += bias[col + lane];
-      if (krow) krow[lane] = from_float<TA>(u);
+      if (krow) krow[lane] = from_float<TA>(u * f);
       else row[col + lane] = from_float<TA>(u * f);
     }
   }
@@ -82,19 +100,22 @@ __global__ void qkv_prepare_kernel(TA* __restrict__ qkv, int ld, const float* __
 extern "C" int blm_qkv_prepare(void* qkv, int dtype, int ld, const float* bias, const float* cos_sin, int rot,
                                const int* positions, const int* token_seq, const int* block_table, int table_width,
                                void* kcache, void* vcache, int page_size, int T, int H, int G, int dk, int dv, int write_kv,
-                               int adjacent, int values_are_keys, const float* q_scale, hipStream_t stream) {
+                               int adjacent, int values_are_keys, const float* q_scale, int unit_norm, float norm_eps,
+                               hipStream_t stream) {
   BLM_REQUIRE(T > 0 && H > 0 && G > 0 && dk > 0 && dv > 0, "qkv_prepare: bad sizes T=%d H=%d G=%d dk=%d dv=%d", T, H, G, dk, dv);
   BLM_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dk, "qkv_prepare: %d turning lanes of %d (even, at most the head size)", rot, dk);
   BLM_REQUIRE(!values_are_keys || dv == dk, "qkv_prepare: values that are the keys have the keys' head size, not %d", dv);
   BLM_REQUIRE(ld >= H * dk + (write_kv ? G * (dk + (values_are_keys ? 0 : dv)) : 0), "qkv_prepare: rows of %d are too short", ld);
   BLM_REQUIRE(!write_kv || (kcache && vcache && block_table && page_size > 0 && table_width > 0), "qkv_prepare: the pages are missing");
   BLM_REQUIRE(rot == 0 || cos_sin, "qkv_prepare: the table of angles is missing");
+  const size_t factors = unit_norm ? (size_t)(H + G) * sizeof(float) : 0;
+  BLM_REQUIRE(factors <= 60 * 1024, "qkv_prepare: %d heads are too many", H + G);
   if (dtype == BLM_F32)
-    hipLaunchKernelGGL(qkv_prepare_kernel<float>, dim3(T), dim3(256), 0, stream, (float*)qkv, ld, bias, cos_sin, rot, positions,
-                       token_seq, block_table, table_width, (float*)kcache, (float*)vcache, page_size, H, G, dk, dv, write_kv, adjacent, values_are_keys, q_scale);
+    hipLaunchKernelGGL(qkv_prepare_kernel<float>, dim3(T), dim3(256), factors, stream, (float*)qkv, ld, bias, cos_sin, rot, positions,
+                       token_seq, block_table, table_width, (float*)kcache, (float*)vcache, page_size, H, G, dk, dv, write_kv, adjacent, values_are_keys, q_scale, unit_norm, norm_eps);
   else if (dtype == BLM_BF16)
-    hipLaunchKernelGGL(qkv_prepare_kernel<bf16>, dim3(T), dim3(256), 0, stream, (bf16*)qkv, ld, bias, cos_sin, rot, positions,
-                       token_seq, block_table, table_width, (bf16*)kcache, (bf16*)vcache, page_size, H, G, dk, dv, write_kv, adjacent, values_are_keys, q_scale);
+    hipLaunchKernelGGL(qkv_prepare_kernel<bf16>, dim3(T), dim3(256), factors, stream, (bf16*)qkv, ld, bias, cos_sin, rot, positions,
+                       token_seq, block_table, table_width, (bf16*)kcache, (bf16*)vcache, page_size, H, G, dk, dv, write_kv, adjacent, values_are_keys, q_scale, unit_norm, norm_eps);
   else
     return blm_fail("qkv_prepare: unsupported dtype %d", dtype);
   BLM_LAUNCH_CHECK("qkv_prepare");
@@ -164,7 +185,7 @@ __global__ void sink_attn_kernel(const TA* __restrict__ q, int ldq, float* __res
                                  const int* __restrict__ positions, const int* __restrict__ token_seq,
                                  const int* __restrict__ block_table, int table_width, const TA* __restrict__ kcache,
                                  const TA* __restrict__ vcache, int page_size, int T, int H, int G, int dk, int dv,
-                                 float scale, int window, int all_groups) {
+                                 float scale, int window, int all_groups, int keep_first, float cap) {
   extern __shared__ float sa_sm[];
   const int waves = blockDim.x / BLM_WAVE;
   const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
@@ -200,9 +221,12 @@ __global__ void sink_attn_kernel(const TA* __restrict__ q, int ldq, float* __res
 #pragma unroll
     for (int i = 0; i < SA_MAX_DV_REGS; ++i) acc[c][i] = 0.f;
 
-  for (int j0 = first; j0 <= pos; j0 += BLM_WAVE) {
-    const int j = j0 + lane;
-    const bool valid = j <= pos;
+  // the keys seen are those of the window and, before it, the sequence's first keep_first: walked as one list
+  const int kept = min(keep_first, first), n_seen = kept + pos - first + 1;
+  for (int x0 = 0; x0 < n_seen; x0 += BLM_WAVE) {
+    const int x = x0 + lane;
+    const int j = x < kept ? x : first + x - kept;
+    const bool valid = x < n_seen;
     float s = -INFINITY;
     int page = 0, in_page = 0;
     if (valid) {
@@ -212,13 +236,14 @@ __global__ void sink_attn_kernel(const TA* __restrict__ q, int ldq, float* __res
       float dot = 0.f;
       for (int d = 0; d < dk; ++d) dot = fmaf(qs[d], to_float(krow[d]), dot);
       s = dot * scale;
+      if (cap > 0.f) s = cap * tanhf(s / cap);
     }
     const float m_new = fmaxf(m, wave_max(s));
     const float p = valid ? expf(s - m_new) : 0.f;
     const float corr = expf(m - m_new);      // m is finite with a sink; without one, -inf only before the first chunk
     l = l * corr + wave_sum(p);
     m = m_new;
-    const int cnt = (pos - j0 + 1) < BLM_WAVE ? (pos - j0 + 1) : BLM_WAVE;
+    const int cnt = (n_seen - x0) < BLM_WAVE ? (n_seen - x0) : BLM_WAVE;
 #pragma unroll
     for (int c = 0; c < GB; ++c) {
       const int cc = c0 + c;
@@ -299,7 +324,8 @@ static int launch_talk_mix(const float* A, const float* mix, void* out, int dtyp
 extern "C" int blm_sink_attn(const void* q, int ldq, void* out, int dtype, float* A, const float* sinks, const float* mix,
                              const int* positions, const int* token_seq, const int* block_table, int table_width,
                              const void* kcache, const void* vcache, int page_size, int T, int H, int G, int dk, int dv,
-                             float scale, int window, hipStream_t stream) {
+                             float scale, int window, int keep_first, float cap, hipStream_t stream) {
+  BLM_REQUIRE(keep_first >= 0 && cap >= 0.f, "sink_attn: keep_first %d or cap %g is negative", keep_first, (double)cap);
   BLM_REQUIRE(T > 0 && H > 0 && G > 0 && H % G == 0, "sink_attn: bad sizes T=%d heads=%d kv_heads=%d", T, H, G);
   BLM_REQUIRE(dk > 0 && dk <= SA_MAX_DK && dv > 0 && dv <= 64 * SA_MAX_DV_REGS,
               "sink_attn: head sizes %d / %d are not supported (keys up to %d, values up to %d)", dk, dv, SA_MAX_DK, 64 * SA_MAX_DV_REGS);
@@ -318,7 +344,7 @@ extern "C" int blm_sink_attn(const void* q, int ldq, void* out, int dtype, float
 #define SA_CASE(TA, GB)                                                                                               \
   hipLaunchKernelGGL((sink_attn_kernel<TA, GB>), grid, block, per_wave * waves, stream, (const TA*)q, ldq, A, sinks, \
                      positions, token_seq, block_table, table_width, (const TA*)kcache, (const TA*)vcache, page_size, T, H, G, \
-                     dk, dv, scale, window, all_groups)
+                     dk, dv, scale, window, all_groups, keep_first, cap)
 #define SA_PICK(TA)                  \
   do {                               \
     if (gb == 8) SA_CASE(TA, 8);     \

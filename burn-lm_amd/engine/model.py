@@ -19,6 +19,9 @@ class Model:
         self.embedding = registry.part("embedding", plan.embedding.kind)(plan.embedding.params, plan.embedding.names)
         self.final_norm = registry.part("norm", plan.final_norm.kind)(plan.final_norm.params, plan.final_norm.names)
         self.head = registry.part("head", plan.head.kind)(plan.head.params, plan.head.names)
+        self.entry = registry.part("connection", plan.entry.kind)(plan.entry.params, plan.entry.names) if plan.entry else None
+        if self.entry is None and any(p.turn is not None for p in plan.order):
+            raise ValueError("a place of the layer order starts a pass, but the plan has no entry part")
         self.blocks = []
         for li, lp in enumerate(plan.layers):
             block_cls = registry.part("block", lp.block)
@@ -45,6 +48,8 @@ class Model:
         encoding while it binds its own projections."""
         yield from self.positions.values()
         yield self.embedding
+        if self.entry is not None:
+            yield self.entry
         for b in self.blocks:
             yield from b.parts()
         yield self.final_norm
@@ -89,19 +94,31 @@ class Model:
                 flops += part.step_flops(rows)
                 if hasattr(part, "mixing_flops"):
                     flops += sum(part.mixing_flops(p, n) for p, n in zip(pasts, news))
+            if place.turn is not None:
+                weight_bytes += self.entry.step_bytes(rows)
+                flops += self.entry.step_flops(rows)
         cache_bytes = 0
         if cache is not None:
             cache_bytes = sum(cache.bytes_read(p + n, with_state=True) for p, n in zip(pasts, news))
         return dict(weight_bytes=weight_bytes, cache_bytes=cache_bytes, flops=flops)
 
+    def _embed(self, step, copy):
+        if copy is not None or getattr(self.embedding, "positional", False):
+            return self.embedding.forward_at(step, copy)
+        if step.token_source is None:
+            return self.embedding.forward(step.token_ids)
+        return self.embedding.forward_from(step.token_ids, *step.token_source)
+
     def forward(self, step, cache):
         """Logits (float32, [wanted rows, vocab]) of one step, or None when no row is wanted."""
-        if step.token_source is None:
-            h = self.embedding.forward(step.token_ids)
-        else:
-            h = self.embedding.forward_from(step.token_ids, *step.token_source)
+        both = None      # a loop's rows [x; x0]: the embedding leaves its half there
+        if self.entry is not None:
+            both = self.entry.begin(step.n_tokens, step.token_ids.device)
+        h = self._embed(step, None if both is None else both[:, both.shape[1] // 2:])
         delta = None
         for i, place in enumerate(self.plan.order):
+            if place.turn is not None:
+                delta = self.entry.enter(h, delta, both, place.turn)
             delta = self.blocks[place.layer].forward(h, delta, step, cache.views[i])
         if step.n_wanted == 0:
             return None

@@ -44,6 +44,7 @@ class LayerPlan:
 class Place:
     layer: int
     reads_cache_of: Optional[int] = None  # index of an earlier place in the order
+    turn: Optional[int] = None  # pass t of a loop starts here: the plan's entry runs in front of the layer
 
 
 @dataclass
@@ -57,5 +58,6 @@ class ModelPlan:
     final_norm: PartSpec
     head: PartSpec
     positions: Dict[str, PartSpec] = field(default_factory=dict)
+    entry: Optional[PartSpec] = None  # a connection in front of every pass of a loop (see Place.turn)
     stop_ids: Tuple[int, ...] = ()
     ignorable_tensors: Tuple[str, ...] = ()  # regular expressions of checkpoint names to skip silently

@@ -1,11 +1,12 @@
 """Parts a model is assembled from, and their registration under kind names."""
 from .. import registry
 from .attention import Attention
-from .base import (Block, FeedForward, Gated, KVNeed, Mixer, Norm, Part, PartSpec, PositionEncoding, StateNeed,
+from .base import (Block, FeedForward, Gated, Joining, KVNeed, Mixer, Norm, Part, PartSpec, PositionEncoding, StateNeed,
                    TensorSpec)
 from .block import PreNormBlock
 from .channel_delta import ChannelDelta
 from .clamped_glu import ClampedGLU
+from .dense_relu2 import DenseRelu2
 from .dense_xielu import DenseXielu
 from .embedding import Embedding, LMHead
 from .gated_residual import GatedPreNormBlock, GatedPreNormMixerBlock, ResidualGate
@@ -14,11 +15,14 @@ from .gla import GatedLinearAttention
 from .hgrn2 import HGRN2
 from .latent_attention import LatentAttention
 from .lightning import LightningAttention
+from .loop import LoopEntry
 from .mixer_pair import MixerPair
+from .mlstm import MLSTM
 from .norm_layer import LayerNorm
 from .norm_rms import RMSNorm
 from .parallel import (CausalConvInput, LayerScale, ParallelBlock, ParallelMixerBlock, ScaledParallelBlock,
                        ScaledParallelMixerBlock, TokenSide)
+from .post_norm import PostNormBlock, PostNormMixerBlock
 from .rope import RotaryEncoding
 from .routed_experts import GroupedRoutedExperts, RoutedExperts
 from .sink_attention import SinkAttention
@@ -58,3 +62,8 @@ registry.register_part("connection", "residual_gate", ResidualGate)
 registry.register_part("block", "pre_norm_gated", GatedPreNormBlock)
 registry.register_part("block", "pre_norm_gated_mixer_only", GatedPreNormMixerBlock)
 registry.register_part("feed_forward", "gelu_glu", GeluGLU)
+registry.register_part("mixer", "mlstm", MLSTM)
+registry.register_part("feed_forward", "dense_relu2", DenseRelu2)
+registry.register_part("block", "post_norm", PostNormBlock)
+registry.register_part("block", "post_norm_mixer_only", PostNormMixerBlock)
+registry.register_part("connection", "loop_entry", LoopEntry)

@@ -13,7 +13,8 @@ Interfaces (all tensors live on the GPU; ``x`` is ``[tokens, width]`` in the act
   the normalised rows (all rows, or the rows listed in ``rows``).  ``delta`` is ``[tokens, width]``
   in the activation dtype, or float32 ``[planes, tokens, width]`` whose planes are summed (a
   mixer or feed-forward may hand on the partial products of its last matrix product), or a ``Gated``
-  (such a result with the gate it joins the residual behind; the RMS norm takes it).
+  (such a result with the gate it joins the residual behind; the RMS norm takes it), or a ``Joining`` (results
+  that are normed before they join, or that the residual starts anew from; the RMS norm takes it).
 * ``Mixer.cache_need() -> KVNeed | StateNeed | None`` and
   ``Mixer.forward(x, step, view) -> delta``; ``view`` is what the cache holds for this place
   in the layer order (``KVView``, ``StateView`` or ``None``).
@@ -33,7 +34,7 @@ Interfaces (all tensors live on the GPU; ``x`` is ``[tokens, width]`` in the act
 from __future__ import annotations
 
 from dataclasses import dataclass, field
-from typing import Dict, Tuple
+from typing import Dict, List, Tuple
 
 import torch
 
@@ -55,7 +56,8 @@ class PartSpec:
 
 @dataclass(frozen=True)
 class KVNeed:
-    """Keys and values per token.  window = 0 keeps every key; window = w keeps the last w.  Values
+    """Keys and values per token.  window = 0 keeps every key; window = w keeps the last w and, beside them, a
+    sequence's first keep_first keys.  Values
     may have a head size of their own (value_dim; 0: that of the keys) and a head count of their own
     (n_value_heads; 0: that of the keys); the attention of this library asks for equal ones.  no_values: there
     are no value pages at all (a mixer whose values are part of its key rows)."""
@@ -65,6 +67,7 @@ class KVNeed:
     value_dim: int = 0
     n_value_heads: int = 0
     no_values: bool = False
+    keep_first: int = 0
 
     @property
     def v_dim(self):
@@ -86,10 +89,14 @@ class StateNeed:
 class Term:
     """One summand of a sublayer's result, for a block that adds the summands to the residual itself (in float32, each
     with coefficients of its own): ``scale * row[t] * y[t, :]``.  y: [tokens, width] in the activation dtype, or float32
-    planes [planes, tokens, width] that are summed; row: float32 [tokens] (any stride) or None."""
+    planes [planes, tokens, width] that are summed; row: float32 [tokens] (any stride) or None.  gamma (float32 [width]
+    or None): y is RMS-normed over its width with this weight and eps before the scale (only for a block that joins its
+    results as a Joining)."""
     y: torch.Tensor
     scale: float = 1.0
     row: torch.Tensor = None
+    gamma: torch.Tensor = None
+    eps: float = 0.0
 
 
 @dataclass
@@ -102,6 +109,19 @@ class Gated:
     z: torch.Tensor
     bias: torch.Tensor = None
     mult: float = 1.0
+
+
+@dataclass
+class Joining:
+    """What joins the residual at the next norm, with work of its own on the way: the sum of the terms, RMS-normed with
+    gamma (float32 [width]) and eps where gamma is given; plus vec (float32 [width]) where given.  fresh: the residual
+    starts anew from this instead of growing by it.  A norm takes it where it takes a plain delta and does all of it, the
+    add and its own work in one kernel."""
+    terms: List[Term]
+    gamma: torch.Tensor = None
+    eps: float = 0.0
+    fresh: bool = False
+    vec: torch.Tensor = None
 
 
 class Part:

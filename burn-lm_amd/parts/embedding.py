@@ -6,6 +6,8 @@ A tied head uses the embedding table itself: the ``[vocab, width]`` table is the
 ``[d_out, d_in]`` matrix (the reference leaves tying as a TODO, transformer.rs:82-84)."""
 from __future__ import annotations
 
+import math
+
 import torch
 
 from .base import Part, TensorSpec
@@ -13,7 +15,9 @@ from .base import Part, TensorSpec
 
 class Embedding(Part):
     """params: vocab, width, copies (default 1; more: the residual starts as that many equal streams,
-    [tokens, copies, width]), scale (default 1: every row is multiplied by it).  names: weight."""
+    [tokens, copies, width]), scale (default 1: every row is multiplied by it), position_base (default none; a number b: a
+    sinusoidal vector of the token's position p is added, entry 2i the sine and entry 2i + 1 the cosine of
+    p * b^(-2i/width); the angles are reduced in double precision).  names: weight."""
     graph_safe = True
 
     def tensor_specs(self):
@@ -23,6 +27,15 @@ class Embedding(Part):
         self.rt = rt
         self.table = tensors[self.names["weight"]].contiguous()
         self.scale = float(self.params.get("scale", 1.0))
+        base, d = self.params.get("position_base"), self.params["width"]
+        self.turns = None      # full turns of entries 2i and 2i + 1 per position
+        if base is not None:
+            exponents = torch.arange((d + 1) // 2, dtype=torch.float64) * (-2.0 / d)
+            self.turns = (float(base) ** exponents / (2.0 * math.pi)).to(rt.device)
+
+    @property
+    def positional(self):
+        return self.params.get("position_base") is not None
 
     def step_bytes(self, rows):
         return rows * self.params["width"] * self.table.element_size()      # the rows that are looked up
@@ -32,7 +45,17 @@ class Embedding(Part):
         shape = (ids.shape[0], self.params["width"]) if copies == 1 else (ids.shape[0], copies, self.params["width"])
         return torch.empty(shape, dtype=torch.float32, device=ids.device)
 
+    def forward_at(self, step, copy=None):
+        """The rows of a step's tokens with their positions' vectors; copy (a view [tokens, width] in the activation
+        dtype) receives them once more."""
+        if int(self.params.get("copies", 1)) != 1 or self.scale != 1.0:
+            raise ValueError("positions' vectors and copies of the embedding come with one unscaled stream")
+        return self.rt.ops.embed_positions(self.table, step.token_ids, step.positions, self.turns, self._rows(step.token_ids),
+                                           copy=copy, source=step.token_source)
+
     def forward(self, ids):
+        if self.positional:
+            raise ValueError("an embedding with positions' vectors needs the step: forward_at")
         h = self._rows(ids)
         return self.rt.ops.embed_gather(self.table, ids, h, self.scale)
 

@@ -90,9 +90,18 @@ class GroupedRoutedExperts(RoutedExperts):
     ``identity`` of the router's outputs belong to experts without tensors that hand their input on unchanged; they
     count like the others in softmax, groups and choice, and their share of the result is ``weight * x``.
 
+    Variants by parameter: scores that are each expert's own sigmoid (``score="sigmoid"``); weights that are the chosen
+    scores as they are (``renormalize=False``); clamped experts (``form="clamped"``) whose weight is on their input: an
+    expert reads ``w x``, ``g = min(W_gate (w x), limit)``, ``u = clamp(W_up (w x), -limit, limit)`` and gives
+    ``W_down (g sigmoid(alpha g) (u + 1))``; with them a shared expert of the same form, with a limit of its own, that runs
+    for every token unweighted.  The share on the input goes through the stacked product as a factor on its results.
+
     params: width, experts (those with tensors), identity (default 0), top, groups (default 1), keep (default 1),
-    expert_inner, correction (whether the checkpoint has one; default True).
-    names: router [experts + identity, width], correction [experts + identity], e<i>.gate / e<i>.up / e<i>.down."""
+    expert_inner, correction (whether the checkpoint has one; default True), score ("softmax", the default, or "sigmoid"),
+    renormalize (default True), form ("silu", the default, or "clamped"; then limit, alpha (default 1.702), shared_inner
+    (default 0: no shared expert), shared_limit).
+    names: router [experts + identity, width], correction [experts + identity], e<i>.gate / e<i>.up / e<i>.down, and with a
+    shared expert shared.gate / shared.up / shared.down."""
 
     def _counts(self):
         p = self.params
@@ -102,6 +111,9 @@ class GroupedRoutedExperts(RoutedExperts):
             raise ValueError(f"grouped experts: {E} + {I} experts do not form {groups} equal groups of which {keep} stay")
         if not 1 <= p["top"] <= keep * ((E + I) // groups):
             raise ValueError(f"grouped experts: top = {p['top']} is more than {keep} groups of {(E + I) // groups} hold")
+        form = p.get("form", "silu")
+        if form not in ("silu", "clamped") or (form == "silu" and p.get("shared_inner")):
+            raise ValueError(f"grouped experts: form {form!r} unknown (silu, clamped), or a shared expert that is not clamped")
         return E, I, groups, keep
 
     def tensor_specs(self):
@@ -115,19 +127,27 @@ class GroupedRoutedExperts(RoutedExperts):
             specs[n[f"e{e}.gate"]] = TensorSpec((f, d))
             specs[n[f"e{e}.up"]] = TensorSpec((f, d))
             specs[n[f"e{e}.down"]] = TensorSpec((d, f))
+        s = int(p.get("shared_inner", 0))
+        if s:
+            specs.update({n["shared.gate"]: TensorSpec((s, d)), n["shared.up"]: TensorSpec((s, d)), n["shared.down"]: TensorSpec((d, s))})
         return specs
 
     def bind(self, tensors, rt):
         self.rt = rt
         p, n = self.params, self.names
         self.E, self.I, self.groups, self.keep = self._counts()
-        self.top, self.f, self.s = int(p["top"]), p["expert_inner"], 0
+        self.top, self.f, self.s = int(p["top"]), p["expert_inner"], int(p.get("shared_inner", 0))
+        self.score, self.renormalize = p.get("score", "softmax"), bool(p.get("renormalize", True))
+        self.clamped = p.get("form", "silu") == "clamped"
+        if self.clamped:
+            self.limit, self.alpha = float(p["limit"]), float(p.get("alpha", 1.702))
+            self.shared_limit = float(p["shared_limit"]) if self.s else None
         t = lambda name: tensors[n[name]]
-        gates, ups = [t(f"e{e}.gate") for e in range(self.E)], [t(f"e{e}.up") for e in range(self.E)]
-        downs = [t(f"e{e}.down") for e in range(self.E)]
+        blocks = [f"e{e}." for e in range(self.E)] + (["shared."] if self.s else [])
+        gates, ups, downs = ([t(b + r) for b in blocks] for r in ("gate", "up", "down"))
         if len({w.dtype for w in gates + ups + downs}) != 1:
             gates, ups, downs = ([w.float() for w in group] for group in (gates, ups, downs))
-        self.inner = self.E * self.f
+        self.inner = self.E * self.f + self.s
         self.w_gate_up = rt.weight(torch.cat(gates + ups, dim=0))
         self.w_down = rt.weight(torch.cat(downs, dim=1).contiguous())
         router = t("router")
@@ -143,14 +163,19 @@ class GroupedRoutedExperts(RoutedExperts):
         rt = self.rt
         logits = rt.linear(x, self.w_router, out_dtype=torch.float32)
         weights = torch.empty(x.shape[0], self.E + 1, dtype=torch.float32, device=x.device)
-        return rt.ops.moe_route_grouped(logits, self.correction, self.E, self.I, self.groups, self.keep, self.top, weights)
+        return rt.ops.moe_route_grouped(logits, self.correction, self.E, self.I, self.groups, self.keep, self.top, weights,
+                                        score=self.score, renormalize=self.renormalize)
 
     def forward_terms(self, x, step):
         rt = self.rt
         weights = self.route(x)
         gu = rt.linear(x, self.w_gate_up)
         act = torch.empty(x.shape[0], self.inner, dtype=gu.dtype, device=x.device)
-        terms = [Term(rt.linear(rt.ops.moe_gate(gu, weights, act, self.E, self.f), self.w_down, partials=True))]
+        if self.clamped:
+            rt.ops.moe_gate_clamped(gu, weights, act, self.E, self.f, self.limit, self.alpha, self.shared_limit)
+        else:
+            rt.ops.moe_gate(gu, weights, act, self.E, self.f)
+        terms = [Term(rt.linear(act, self.w_down, partials=True))]
         if self.I:
             terms.append(Term(x, 1.0, weights[:, self.E]))
         return terms

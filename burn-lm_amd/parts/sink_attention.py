@@ -15,7 +15,10 @@ Variants by parameter: no biases at all (``bias=False``); turning pairs of adjac
 (``values="keys"``; then ``vdim = dim``); a stored temperature per head that multiplies the head's scores
 (``temperature=True``; it rides on the queries, which the scores are linear in, applied in float32 behind their
 rotation); an output gate (``gate=True``): the concatenated heads are multiplied element by element by
-``sigmoid(W_g x)`` of the mixer's own input before the output projection (``W_g`` runs with the other projections)."""
+``sigmoid(W_g x)`` of the mixer's own input before the output projection (``W_g`` runs with the other projections);
+queries and keys (with their biases) divided by their root mean square over each head's lanes in front of the rotation
+(``unit_norm_eps``); capped scores ``s <- c tanh(s / c)`` (``softcap``); the first ``keep_first`` keys of a sequence visible
+beside the window, at their true positions (``keep_first``; their pages stay in the cache)."""
 from __future__ import annotations
 
 import os
@@ -33,7 +36,9 @@ class SinkAttention(Mixer):
     the default: lane i turns with lane i + rot_dims/2; "adjacent": lane 2i with 2i + 1), values ("projected", the
     default, or "keys": the unrotated keys are the values and there is no value projection), temperature (whether a
     number per head multiplies its scores; default False), gate (whether the heads pass a sigmoid gate projected from
-    the input; default False).
+    the input; default False), output_bias (whether the output projection has a bias; default: as the others),
+    unit_norm_eps (default none: no norm of queries and keys), softcap (default 0: none), keep_first (default 0; first
+    keys that stay visible beside a window).
     names: q, q_bias, o, o_bias, sink, talk, temp, g and, unless the layer borrows, k, k_bias, v, v_bias (those the
     parameters leave)."""
     graph_safe = True
@@ -70,13 +75,15 @@ class SinkAttention(Mixer):
             specs[n["k"]] = TensorSpec((G * dk, d))
             if not values_are_keys:
                 specs[n["v"]] = TensorSpec((G * dv, d))
-        if bias:
-            specs.update({n[r + "_bias"]: TensorSpec(specs[n[r]].shape[:1]) for r in ("q", "o", "k", "v") if n.get(r) in specs})
+        biased = (("q", "k", "v") if bias else ()) + (("o",) if p.get("output_bias", bias) else ())
+        specs.update({n[r + "_bias"]: TensorSpec(specs[n[r]].shape[:1]) for r in biased if n.get(r) in specs})
         return specs
 
     def cache_need(self):
         p = self.params
-        return KVNeed(p["kv_heads"], p["dim"], int(p.get("cache_window", p.get("window", 0))), value_dim=p["vdim"])
+        window = int(p.get("cache_window", p.get("window", 0)))
+        return KVNeed(p["kv_heads"], p["dim"], window, value_dim=p["vdim"],
+                      keep_first=int(p.get("keep_first", 0)) if window > 0 else 0)
 
     def bind(self, tensors, rt):
         self.rt = rt
@@ -85,6 +92,12 @@ class SinkAttention(Mixer):
         if self.H % self.G:
             raise ValueError(f"{self.H} heads are no multiple of {self.G} key-value heads")
         self.scale, self.window, self.rot = float(p["scale"]), int(p.get("window", 0)), int(p.get("rot_dims", 0))
+        self.keep_first = int(p.get("keep_first", 0)) if self.window > 0 else 0
+        self.softcap = float(p.get("softcap") or 0.0)
+        eps = p.get("unit_norm_eps")
+        self.unit_norm_eps = None if eps is None else float(eps)
+        if self.softcap < 0.0 or self.keep_first < 0:
+            raise ValueError("sink attention: softcap and keep_first are not negative")
         self.borrows, sink, talk = self._flags()
         bias, self.values_are_keys, self.adjacent = self._variant()
         self.position = p.get("position")
@@ -110,7 +123,7 @@ class SinkAttention(Mixer):
         self.w_in = rt.weight(torch.cat(ws, dim=0))
         self.bias_in = torch.cat([tensors[n[r + "_bias"]].float() for r in roles]).contiguous() if bias else None
         self.w_o = rt.weight(tensors[n["o"]])
-        self.output_bias = tensors[n["o_bias"]].float().contiguous() if bias else None
+        self.output_bias = tensors[n["o_bias"]].float().contiguous() if p.get("output_bias", bias) else None
         self.on_matrix_cores = rt.ops.sink_attn_mfma_supported(rt.dtype, self.dk, self.dv) and self.scale > 0 \
             and os.environ.get("BURN_LM_AMD_SINK_ATTENTION") != "generic"
         # without head mixing and with values of the keys' size this is the plain attention's arithmetic plus a share of
@@ -118,6 +131,13 @@ class SinkAttention(Mixer):
         self.on_plain_kernels = self.on_matrix_cores and not talk and self.dk == self.dv \
             and rt.ops.attn_decode_supported(rt.dtype, self.dk) and rt.ops.attn_prefill_mfma_supported(rt.dtype, self.dk) \
             and os.environ.get("BURN_LM_AMD_SINK_ATTENTION") != "own"
+        # caps and first keys: the plain attention's kernels (which do not ask for the other form's head sizes) or the
+        # generic kernel
+        if self.softcap > 0.0 or self.keep_first > 0:
+            self.on_matrix_cores = False
+            self.on_plain_kernels = not talk and self.dk == self.dv and self.scale > 0 \
+                and rt.ops.attn_decode_supported(rt.dtype, self.dk) and rt.ops.attn_prefill_mfma_supported(rt.dtype, self.dk) \
+                and os.environ.get("BURN_LM_AMD_SINK_ATTENTION") != "generic"
         if self.on_matrix_cores:
             rt.ops.latent_attn_init(rt.device)     # the pieces' workspace, before any step is recorded
             rt.ops.sink_attn_mfma_init(rt.device)  # likewise: the shared memory of the form that stages pages
@@ -133,7 +153,7 @@ class SinkAttention(Mixer):
 
     def mixing_flops(self, past, new):
         """Scores once, weighted values once for every key-value head (the mixing is done behind the sum over keys)."""
-        keys = sum(min(past + t + 1, self.window) if self.window else past + t + 1 for t in range(new)) if self.window \
+        keys = sum(min(past + t + 1, self.window + self.keep_first) for t in range(new)) if self.window \
             else new * past + new * (new + 1) // 2
         return 2 * self.H * (self.dk + self.dv * (self.G if self.talk is not None else 1)) * keys
 
@@ -166,7 +186,7 @@ class SinkAttention(Mixer):
         rt.ops.qkv_prepare(qkv, self.bias_in, self.position.table if self.rot else None, self.rot, step,
                            view.block_table(step), view.k, view.v, view.page_size, self.H, self.G, self.dk, self.dv,
                            write_kv=store, adjacent=self.adjacent, values_are_keys=self.values_are_keys,
-                           q_scale=self.temperature)
+                           q_scale=self.temperature, unit_norm_eps=self.unit_norm_eps)
         return qkv
 
     def attend(self, qkv, step, view):
@@ -201,7 +221,8 @@ class SinkAttention(Mixer):
                                          view.page_size, self.H, self.G, self.dk, self.dv, self.scale, self.window,
                                          n_splits=n_splits, group_batch=group_batch)
         return rt.ops.sink_attn(qkv, out, self.sinks, self.talk, step, view.block_table(step), view.k, view.v,
-                                view.page_size, self.H, self.G, self.dk, self.dv, self.scale, self.window)
+                                view.page_size, self.H, self.G, self.dk, self.dv, self.scale, self.window,
+                                keep_first=self.keep_first, softcap=self.softcap)
 
     def _attend_plain(self, qkv, out, step, view):
         """The plain attention's kernels (decode: key ranges cut as that mixer cuts them), with the sink."""
@@ -210,18 +231,18 @@ class SinkAttention(Mixer):
         H, G, hd = self.H, self.G, self.dk
         if step.max_new == 1:
             span = step.max_len_after if not self.window else min(step.max_len_after, self.window + view.page_size)
-            pages = (span + view.page_size - 1) // view.page_size
+            pages = (span + view.page_size - 1) // view.page_size + -(-self.keep_first // view.page_size)
             blocks = qkv.shape[0] * G * ((H // G + 15) // 16)
             rt.ops.attn_decode(qkv, qkv.stride(0), out, step.positions, step.token_seq, table, view.k, view.v, view.page_size,
                                H, G, hd, self.scale, self.window, decode_splits(pages, blocks, hd, rt.compute_units),
-                               sinks=self.sinks)
+                               sinks=self.sinks, keep_first=self.keep_first, softcap=self.softcap)
         else:
             queries = rt.prefill_queries or rt.ops.attn_prefill_queries(step.n_seqs, step.max_new, H, G, hd, rt.compute_units)
             if queries == 32 and (hd % 32 or hd > 128):
                 queries = 16
             rt.ops.attn_prefill_mfma(qkv, qkv.stride(0), out, step.positions, step.cu_seqlens, table, view.k, view.v,
                                      view.page_size, step.n_seqs, step.max_new, H, G, hd, self.scale, self.window,
-                                     queries=queries, sinks=self.sinks)
+                                     queries=queries, sinks=self.sinks, keep_first=self.keep_first, softcap=self.softcap)
         return out
 
     def output(self, attended):

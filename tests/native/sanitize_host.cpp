@@ -55,7 +55,7 @@ struct Rng {
 
 // No page lost, none held twice, tables as long as the lengths say, windows give back what fell out.
 static void check_books(BlmCache* c, const std::map<int, int>& live, int page, const int* n_pages, const int* windows,
-                        int n_groups) {
+                        const int* keep, int n_groups) {
   for (int g = 0; g < n_groups; ++g) {
     BlmPool* pool = blm_cache_pool(c, g);
     std::vector<int> free_list(n_pages[g]);
@@ -71,7 +71,7 @@ static void check_books(BlmCache* c, const std::map<int, int>& live, int page, c
       CHECK(blm_cache_table(c, g, slot, table.data()) == BLM_OK);
       const int first_key = windows[g] ? std::max(0, len - windows[g] + 1) : 0;
       for (int i = 0; i < tl; ++i) {
-        const bool held = i >= first_key / page;
+        const bool held = i >= first_key / page || i * page < keep[g];
         CHECK((table[i] >= 0) == held);
         if (table[i] >= 0) {
           CHECK(table[i] < n_pages[g]);
@@ -86,9 +86,9 @@ static void check_books(BlmCache* c, const std::map<int, int>& live, int page, c
 
 static void cache_traffic(uint64_t seed) {
   Rng rnd(seed);
-  const int page = 16, n_groups = 2, max_seqs = 5, max_context = 96;
-  const int n_pages[2] = {20, 20}, windows[2] = {0, 24};
-  BlmCache* c = blm_cache_new(n_groups, n_pages, windows, page, max_seqs, max_context);
+  const int page = 16, n_groups = 3, max_seqs = 5, max_context = 96;
+  const int n_pages[3] = {20, 20, 20}, windows[3] = {0, 24, 24}, keep[3] = {0, 0, 20};
+  BlmCache* c = blm_cache_new(n_groups, n_pages, windows, keep, page, max_seqs, max_context);
   CHECK(c != nullptr);
   std::map<int, int> live;
   const int growths[5] = {1, 1, 1, 7, 30};
@@ -123,7 +123,7 @@ static void cache_traffic(uint64_t seed) {
         for (size_t i = 0; i < slots.size(); ++i) live[slots[i]] += grow[i];
       }
     }
-    check_books(c, live, page, n_pages, windows, n_groups);
+    check_books(c, live, page, n_pages, windows, keep, n_groups);
     // every fourth move: the live sequences' next step, assembled with and without padding
     if (move % 4 == 0 && !live.empty()) {
       std::vector<int> slots, counts, tokens, want_counts, wants;
@@ -173,7 +173,7 @@ static void cache_traffic(uint64_t seed) {
           if (width > 1) CHECK(blm_cache_page_table(c, 0, n, slots.data(), width - 1, table.data()) == BLM_E_USAGE);
           CHECK(blm_cache_advance_all(c, n, slots.data(), counts.data()) == BLM_OK);
           for (int i = 0; i < n; ++i) live[slots[i]] += counts[i];
-          check_books(c, live, page, n_pages, windows, n_groups);
+          check_books(c, live, page, n_pages, windows, keep, n_groups);
         }
       }
     }
@@ -185,7 +185,7 @@ static void cache_traffic(uint64_t seed) {
   CHECK(blm_cache_reserve(c, 1, &slot, &one, detail) == BLM_E_USAGE);
   for (const auto& [s, len] : live) CHECK(blm_cache_close(c, s) == BLM_OK);
   live.clear();
-  check_books(c, live, page, n_pages, windows, n_groups);
+  check_books(c, live, page, n_pages, windows, keep, n_groups);
   CHECK(blm_cache_n_free_slots(c) == max_seqs);
   for (int g = 0; g < n_groups; ++g) CHECK(blm_pool_n_free(blm_cache_pool(c, g)) == n_pages[g]);
   blm_cache_free(c);

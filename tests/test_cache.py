@@ -81,6 +81,31 @@ def test_groups_with_different_needs_have_storage_and_pools_of_their_own():
     check_invariants(c)
 
 
+def test_first_keys_kept_beside_a_window_keep_their_pages():
+    c = make([KVNeed(2, 8, window=20), KVNeed(2, 8, window=20, keep_first=17), KVNeed(2, 8, keep_first=17)])
+    assert len(c.groups) == 3      # what is kept is part of the need
+    plain, kept = c.groups[0], c.groups[1]
+    s = c.open()
+    c.reserve([(s, 70)]); c.advance(s, 70)
+    assert kept.kept_pages == 2 and c.groups[2].kept_pages == 0
+    assert plain.tables[s][:3] == [-1, -1, -1] and all(p >= 0 for p in plain.tables[s][3:])
+    assert kept.tables[s][2] == -1 and all(p >= 0 for p in kept.tables[s][:2] + kept.tables[s][3:])
+    assert all(p >= 0 for p in c.groups[2].tables[s])
+    first = kept.tables[s][:2]
+    for _ in range(20):            # the same pages for as long as the sequence lives
+        c.reserve([(s, 1)]); c.advance(s, 1)
+    assert kept.tables[s][:2] == first and kept.tables[s][2:4] == [-1, -1] and kept.tables[s][5] >= 0
+    assert c.bytes_read(90) > c.bytes_read(20)
+    c.close(s)
+    assert c.pages_in_use() == 0
+    # a sequence that ends inside its first keys
+    s = c.open()
+    c.reserve([(s, 5)]); c.advance(s, 5)
+    assert len([p for p in kept.tables[s] if p >= 0]) == 1
+    c.close(s)
+    assert c.pages_in_use() == 0
+
+
 def test_a_place_may_read_an_earlier_places_cache():
     c = make([KVNeed(2, 8), KVNeed(2, 8), KVNeed(2, 8)], [None, None, 0])
     assert c.groups[0].k_storage.shape[0] == 2
