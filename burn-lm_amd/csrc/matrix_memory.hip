@@ -18,7 +18,8 @@
 //   A_ts = (q_t . k_s) exp(F_t - F_s + i_s - m_t) for s <= t;   c_t = exp(F_t + m_in - m_t)
 //   o_t = (sum_s A_ts v_s + c_t S_in^T q_t) / (max(|sum_s A_ts + c_t n_in . q_t|, exp(-m_t)) + 1e-6)
 //   S_out = c_n S_in + sum_s exp(F_n - F_s + i_s - m_n) k_s v_s^T,  n_out likewise
-// All exponents are at most zero.  Kernels: mm_gates (a wavefront per (sequence, head) walks the chunks: prefix sums
+// All exponents are at most zero.  F is double: a head that forgets fast reaches sums of several hundred within a chunk,
+// and the difference of two of them is the logarithm of a weight.  Kernels: mm_gates (a wavefront per (sequence, head) walks the chunks: prefix sums
 // and prefix maxima over the 64 lanes), mm_state (each chunk's own share of S and n), mm_carry (the chunks' start
 // states in order), mm_out, then the norm.  Matrix instruction layouts as for lightning attention (recurrent.hip).
 #include "chunk_form.h"
@@ -183,11 +184,12 @@ extern "C" int blm_mm_step(const void* proj, int proj_dtype, int ld, const float
 }
 
 // ---- prompts ------------------------------------------------------------------------------------------
-// gates [3][H][T] float: F (the chunk's running sum of log f), log i, m; chunk [B][n_seg][H][2] float: m at the chunk's
+// sums [H][T] double: F (the chunk's running sum of log f); gates [2][H][T] float: log i, m; chunk [B][n_seg][H][2] float: m at the chunk's
 // start, and c_n, what the chunk leaves of its start state.  Leaves the sequence's m.
 __global__ void __launch_bounds__(BLM_WAVE)
     mm_gates_kernel(const float* __restrict__ z, int ldz, const float* __restrict__ bias_i, const float* __restrict__ bias_f,
-                    float cap, float* __restrict__ gates, float* __restrict__ chunk, float* __restrict__ m_state,
+                    float cap, double* __restrict__ sums, float* __restrict__ gates, float* __restrict__ chunk,
+                    float* __restrict__ m_state,
                     const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slots, int T, int H, int n_seg) {
   const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x;
   const int slot = seq_slots[b], first = cu_seqlens[b], n_new = cu_seqlens[b + 1] - first;
@@ -206,31 +208,32 @@ __global__ void __launch_bounds__(BLM_WAVE)
     const bool valid = t0 + lane < n_new;
     const MmGates g = mm_gates(zi + bi, zf + bf, cap, inv_cap);
     fetch(t0 + LC_CHUNK + lane);      // the next chunk's logits travel meanwhile
-    float F = valid ? g.log_f : 0.f;
+    double F = valid ? (double)g.log_f : 0.0;
 #pragma unroll
     for (int d = 1; d < BLM_WAVE; d <<= 1) {
-      const float o = __shfl_up(F, d, BLM_WAVE);
+      const double o = __shfl_up(F, d, BLM_WAVE);
       if (lane >= d) F += o;
     }
-    float top = valid ? g.log_i - F : -INFINITY;
+    double top = valid ? (double)g.log_i - F : -1e300;
 #pragma unroll
     for (int d = 1; d < BLM_WAVE; d <<= 1) {
-      const float o = __shfl_up(top, d, BLM_WAVE);
-      if (lane >= d) top = fmaxf(top, o);
+      const double o = __shfl_up(top, d, BLM_WAVE);
+      if (lane >= d) top = fmax(top, o);
     }
-    const float m = F + fmaxf(m_in, top);
+    const float m = (float)(F + fmax((double)m_in, top));
     if (valid) {
       const size_t at = (size_t)h * T + first + t0 + lane;
-      gates[at] = F;
-      gates[(size_t)H * T + at] = g.log_i;
-      gates[(size_t)2 * H * T + at] = m;
+      sums[at] = F;
+      gates[at] = g.log_i;
+      gates[(size_t)H * T + at] = m;
     }
     const int last = min(n_new - t0, LC_CHUNK) - 1;
-    const float F_n = __shfl(F, last, BLM_WAVE), m_n = __shfl(m, last, BLM_WAVE);
+    const double F_n = __shfl(F, last, BLM_WAVE);
+    const float m_n = __shfl(m, last, BLM_WAVE);
     if (lane == 0) {
       float* ck = chunk + (((size_t)b * n_seg + c) * H + h) * 2;
       ck[0] = m_in;
-      ck[1] = expf(F_n + m_in - m_n);
+      ck[1] = expf((float)(F_n + (double)m_in - (double)m_n));
     }
     m_in = m_n;
   }
@@ -240,7 +243,8 @@ __global__ void __launch_bounds__(BLM_WAVE)
 // seg_end [B][n_seg][H][dk][dv], seg_n [B][n_seg][H][dk]: what the chunk's own tokens add to S and n by the chunk's end
 template <typename TA>
 __global__ void __launch_bounds__(LC_THREADS)
-    mm_state_kernel(const TA* __restrict__ proj, int ld, const float* __restrict__ gates, float* __restrict__ seg_end,
+    mm_state_kernel(const TA* __restrict__ proj, int ld, const double* __restrict__ sums, const float* __restrict__ gates,
+                    float* __restrict__ seg_end,
                     float* __restrict__ seg_n, const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slots, int T, int H,
                     int dk, int dv, int n_seg, int n_vt) {
   extern __shared__ __attribute__((aligned(16))) unsigned char mm_sm[];
@@ -261,11 +265,11 @@ __global__ void __launch_bounds__(LC_THREADS)
     lc_stage<TA, 2>(proj + (size_t)(first + t0) * ld, ld, n, op);
   }
   if (threadIdx.x < LC_CHUNK) {
-    const float* F = gates + (size_t)h * T + first + t0;
-    const float* I = F + (size_t)H * T;
+    const double* F = sums + (size_t)h * T + first + t0;
+    const float* I = gates + (size_t)h * T + first + t0;
     const float* M = I + (size_t)H * T;
     const int j = threadIdx.x;
-    wj[j] = j < n ? expf(F[n - 1] - F[j] + I[j] - M[n - 1]) : 0.f;
+    wj[j] = j < n ? expf((float)(F[n - 1] - F[j] + (double)(I[j] - M[n - 1]))) : 0.f;
   }
   __syncthreads();
   const size_t chunk_at = ((size_t)b * n_seg + c) * H + h;
@@ -365,8 +369,8 @@ __global__ void mm_carry_kernel(float* __restrict__ seg_end, float* __restrict__
 
 template <typename TA>
 __global__ void __launch_bounds__(LC_THREADS)
-    mm_out_kernel(const TA* __restrict__ proj, int ld, const float* __restrict__ gates, const float* __restrict__ chunk,
-                  const float* __restrict__ seg_start, const float* __restrict__ seg_n, float q_scale, float* __restrict__ o_raw,
+    mm_out_kernel(const TA* __restrict__ proj, int ld, const double* __restrict__ sums, const float* __restrict__ gates,
+                  const float* __restrict__ chunk, const float* __restrict__ seg_start, const float* __restrict__ seg_n, float q_scale, float* __restrict__ o_raw,
                   const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slots, int T, int H, int dk, int dv, int n_seg,
                   int n_vt) {
   extern __shared__ __attribute__((aligned(16))) unsigned char mm_sm[];
@@ -378,9 +382,9 @@ __global__ void __launch_bounds__(LC_THREADS)
   const int v0 = vt * MM_VT, dvt = min(MM_VT, dv - v0);
   const int DKP = (dk + 31) & ~31, DVP = (dvt + 31) & ~31;
   const int SK = DKP + lc_row_pad<TA>();
-  float* As = reinterpret_cast<float*>(mm_sm);                      // [64][65]
-  float* Fs = As + LC_CHUNK * LC_A_LD;                              // [64] F
-  float* Is = Fs + LC_CHUNK;                                        // [64] log i
+  double* Fs = reinterpret_cast<double*>(mm_sm);                    // [64] F
+  float* As = reinterpret_cast<float*>(Fs + LC_CHUNK);              // [64][65]
+  float* Is = As + LC_CHUNK * LC_A_LD;                              // [64] log i
   float* Ms = Is + LC_CHUNK;                                        // [64] m
   float* cs = Ms + LC_CHUNK;                                        // [64] c_t, times q_scale
   float* dn = cs + LC_CHUNK;                                        // [64] one over the denominators
@@ -396,13 +400,14 @@ __global__ void __launch_bounds__(LC_THREADS)
   }
   const size_t chunk_at = ((size_t)b * n_seg + c) * H + h;
   if (threadIdx.x < LC_CHUNK) {
-    const float* F = gates + (size_t)h * T + first + t0;
+    const size_t row = (size_t)h * T + first + t0;
     const int j = threadIdx.x, at = min(j, n - 1);
-    const float fv = F[at], iv = F[(size_t)H * T + at], mv = F[(size_t)2 * H * T + at];
+    const double fv = sums[row + at];
+    const float iv = gates[row + at], mv = gates[(size_t)H * T + row + at];
     Fs[j] = fv;
     Is[j] = iv;
     Ms[j] = mv;
-    cs[j] = expf(fv + chunk[chunk_at * 2] - mv) * q_scale;
+    cs[j] = expf((float)(fv + ((double)chunk[chunk_at * 2] - (double)mv))) * q_scale;
   }
   __syncthreads();
   const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
@@ -421,11 +426,11 @@ __global__ void __launch_bounds__(LC_THREADS)
         sc = __builtin_amdgcn_mfma_f32_32x32x2f32(to_float(qrow[kb + 2 * u]), to_float(krow[kb + 2 * u]), sc, 0, 0, 0);
     }
     const int j = tj * 32 + lr;
-    const float wj = Is[j] - Fs[j];
+    const double wj = (double)Is[j] - Fs[j];
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int i = ti * 32 + 8 * (r / 4) + 4 * lk + (r & 3);
-      As[i * LC_A_LD + j] = (j <= i && i < n) ? sc[r] * q_scale * expf(Fs[i] + wj - Ms[i]) : 0.f;
+      As[i * LC_A_LD + j] = (j <= i && i < n) ? sc[r] * q_scale * expf((float)(Fs[i] + wj - (double)Ms[i])) : 0.f;
     }
   } else {
     // the fourth wavefront: n_in . q of every token, times c_t, a lane per token
@@ -517,7 +522,7 @@ static size_t mm_state_lds(int dk, int dv, int dtype) {
 static size_t mm_out_lds(int dk, int dv, int dtype) {
   const int DKP = (dk + 31) & ~31, DVP = ((dv < MM_VT ? dv : MM_VT) + 31) & ~31;
   const int es = dtype == BLM_F32 ? 4 : 2, SK = DKP + (dtype == BLM_F32 ? 1 : 2);
-  return (size_t)(LC_CHUNK * LC_A_LD + 5 * LC_CHUNK) * sizeof(float) + (size_t)LC_CHUNK * (2 * SK + DVP) * es;
+  return (size_t)(LC_CHUNK * LC_A_LD + 6 * LC_CHUNK) * sizeof(float) + (size_t)LC_CHUNK * (2 * SK + DVP) * es;
 }
 
 #define MM_DEVICES 64
@@ -541,11 +546,11 @@ extern "C" int blm_mm_chunks_supported(int dk, int dv, int dtype) {
   return (dk >= 1 && dk <= MM_MAX_DK && dv >= 1 && mm_state_lds(dk, dv, dtype) <= MM_LDS_LIMIT && mm_out_lds(dk, dv, dtype) <= MM_LDS_LIMIT) ? 1 : 0;
 }
 
-// n_seg: chunks of 64 tokens that cover the longest sequence of the step; gates [3][H][T], chunk [B][n_seg][H][2], seg
+// n_seg: chunks of 64 tokens that cover the longest sequence of the step; sums [H][T] double, gates [2][H][T], chunk [B][n_seg][H][2], seg
 // [B][n_seg][H][dk][dv], seg_n [B][n_seg][H][dk] float; o_raw [T][H*dv] float; token_seq: rows of padding tokens become zero.
 extern "C" int blm_mm_chunks(const void* proj, int dtype, int ld, const float* z, int ldz, const float* bias_i, const float* bias_f,
                              float cap, float q_scale, const float* norm_w, float eps, float* S, float* n_state, float* m_state,
-                             float* gates, float* chunk, float* seg, float* seg_n, float* o_raw, void* out, const int* cu_seqlens,
+                             double* sums, float* gates, float* chunk, float* seg, float* seg_n, float* o_raw, void* out, const int* cu_seqlens,
                              const int* seq_slots, const int* token_seq, int T, int B, int H, int dk, int dv, int max_new, int n_seg,
                              hipStream_t stream) {
   const int n_vt = (dv + MM_VT - 1) / MM_VT;
@@ -557,16 +562,16 @@ extern "C" int blm_mm_chunks(const void* proj, int dtype, int ld, const float* z
   int dev = -1;
   BLM_REQUIRE(hipGetDevice(&dev) == hipSuccess && dev >= 0 && dev < MM_DEVICES && g_mm_ready[dev],
               "mm_chunks: blm_mm_chunks_init has not run on device %d", dev);
-  hipLaunchKernelGGL(mm_gates_kernel, dim3(H, B), dim3(BLM_WAVE), 0, stream, z, ldz, bias_i, bias_f, cap, gates, chunk, m_state,
+  hipLaunchKernelGGL(mm_gates_kernel, dim3(H, B), dim3(BLM_WAVE), 0, stream, z, ldz, bias_i, bias_f, cap, sums, gates, chunk, m_state,
                      cu_seqlens, seq_slots, T, H, n_seg);
   BLM_LAUNCH_CHECK("mm_gates");
   const dim3 grid((unsigned)n_seg, (unsigned)(H * n_vt), (unsigned)B);
   const size_t lds_a = mm_state_lds(dk, dv, dtype), lds_c = mm_out_lds(dk, dv, dtype);
   if (dtype == BLM_F32)
-    hipLaunchKernelGGL(mm_state_kernel<float>, grid, dim3(LC_THREADS), lds_a, stream, (const float*)proj, ld, gates, seg, seg_n,
+    hipLaunchKernelGGL(mm_state_kernel<float>, grid, dim3(LC_THREADS), lds_a, stream, (const float*)proj, ld, sums, gates, seg, seg_n,
                        cu_seqlens, seq_slots, T, H, dk, dv, n_seg, n_vt);
   else
-    hipLaunchKernelGGL(mm_state_kernel<bf16>, grid, dim3(LC_THREADS), lds_a, stream, (const bf16*)proj, ld, gates, seg, seg_n,
+    hipLaunchKernelGGL(mm_state_kernel<bf16>, grid, dim3(LC_THREADS), lds_a, stream, (const bf16*)proj, ld, sums, gates, seg, seg_n,
                        cu_seqlens, seq_slots, T, H, dk, dv, n_seg, n_vt);
   BLM_LAUNCH_CHECK("mm_state");
   const size_t per = (size_t)H * dk * (dv + 1);
@@ -575,10 +580,10 @@ extern "C" int blm_mm_chunks(const void* proj, int dtype, int ld, const float* z
                      dv, n_seg);
   BLM_LAUNCH_CHECK("mm_carry");
   if (dtype == BLM_F32)
-    hipLaunchKernelGGL(mm_out_kernel<float>, grid, dim3(LC_THREADS), lds_c, stream, (const float*)proj, ld, gates, chunk, seg, seg_n,
+    hipLaunchKernelGGL(mm_out_kernel<float>, grid, dim3(LC_THREADS), lds_c, stream, (const float*)proj, ld, sums, gates, chunk, seg, seg_n,
                        q_scale, o_raw, cu_seqlens, seq_slots, T, H, dk, dv, n_seg, n_vt);
   else
-    hipLaunchKernelGGL(mm_out_kernel<bf16>, grid, dim3(LC_THREADS), lds_c, stream, (const bf16*)proj, ld, gates, chunk, seg, seg_n,
+    hipLaunchKernelGGL(mm_out_kernel<bf16>, grid, dim3(LC_THREADS), lds_c, stream, (const bf16*)proj, ld, sums, gates, chunk, seg, seg_n,
                        q_scale, o_raw, cu_seqlens, seq_slots, T, H, dk, dv, n_seg, n_vt);
   BLM_LAUNCH_CHECK("mm_out");
   const char* gate = (const char*)proj + (size_t)(2 * H * dk + H * dv) * (dtype == BLM_F32 ? 4 : 2);

@@ -71,7 +71,7 @@ _SIGNATURES = {
     "blm_mm_chunks_supported": [_c_int, _c_int, _c_int],
     "blm_mm_chunks": [_c_void_p, _c_int, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_float, _c_float, _c_void_p, _c_float,
                       _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
-                      _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+                      _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "blm_sink_attn_mfma_supported": [_c_int, _c_int],
     "blm_sink_attn_mfma": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                            _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
@@ -1458,8 +1458,9 @@ def matrix_memory(proj, logits, bias_i, bias_f, cap, q_scale, norm_w, eps, state
         return out
     n_seg = -(-step.max_new // LIGHTNING_CHUNK)
     f32 = lambda *shape: torch.empty(*shape, dtype=torch.float32, device=proj.device)
-    gates, chunk, seg, seg_n = f32(3, H, T), f32(B, n_seg, H, 2), f32(B, n_seg, H, dk, dv), f32(B, n_seg, H, dk)
-    _call("blm_mm_chunks", *head, gates.data_ptr(), chunk.data_ptr(), seg.data_ptr(), seg_n.data_ptr(), o_raw.data_ptr(),
+    sums = torch.empty(H, T, dtype=torch.float64, device=proj.device)
+    gates, chunk, seg, seg_n = f32(2, H, T), f32(B, n_seg, H, 2), f32(B, n_seg, H, dk, dv), f32(B, n_seg, H, dk)
+    _call("blm_mm_chunks", *head, sums.data_ptr(), gates.data_ptr(), chunk.data_ptr(), seg.data_ptr(), seg_n.data_ptr(), o_raw.data_ptr(),
           out.data_ptr(), step.cu_seqlens.data_ptr(), step.seq_slots.data_ptr(), step.token_seq.data_ptr(), T, B, H, dk, dv,
           step.max_new, n_seg, _stream())
     return out
