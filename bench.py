@@ -380,9 +380,27 @@ def bitonex_config(width, ff, heads, layers, vocab):
                 layers=made)
 
 
-DESIGNS = {"fuvirax": fuvirax_config, "digasun": digasun_config, "girelix": girelix_config, "bitonex": bitonex_config}
+def belelorn_config(width, ff, heads, layers, vocab):
+    """Softmax attention with a window of 1,024 keys beside 4 kept ones (heads of 128 lanes in groups of four, capped scores)
+    beside lightning attention (as many heads of 128 x 128), and matrix memories (half as many heads of 128 x 256), in
+    turn; the feed-forwards in turn dense (two matrices of 1.5 times the Llama's inner size, as many weights) and 12 experts
+    of 512, 4 chosen, with a shared one of 2,048 (as many weights).  The second and third layer run twice, so that as many
+    layers run as the others have."""
+    dense = dict(kind="dense", ff=12288)
+    moe = dict(kind="moe", expert=dict(ff=512, limit=7.0), router=dict(experts=12, top=4), shared=dict(ff=2048, limit=7.0))
+    pair = dict(left=dict(heads=heads, kv_heads=heads // 4, dim=128, vdim=128, scale=128 ** -0.5, softcap=50.0,
+                          mask=dict(size=1024, keep_first=4)),
+                right=dict(heads=heads, dim=128, vdim=128, decay=[1.0 - 2.0 ** -(2 + 6 * h / heads) for h in range(heads)]))
+    memory = dict(heads=heads // 2, dim=128, vdim=256, gate_cap=15.0)
+    made = [dict(type="mlstm", mixer=memory, mlp=dense if i % 4 == 1 else moe) if i % 2 else
+            dict(type="parallel", mixer=pair, mlp=moe if i % 4 == 0 else dense) for i in range(max(3, layers - 2))]
+    return dict(architecture="Belelorn", vocab=vocab, width=width, norm=dict(eps=1e-6), logit_scale=0.5, layers=made,
+                loop=dict(start=1, stop=3, times=2))
+
+
+DESIGNS = {"belelorn": belelorn_config, "fuvirax": fuvirax_config, "digasun": digasun_config, "girelix": girelix_config, "bitonex": bitonex_config}
 # the designs that run beside one (the Llama of equal size always does): the closest of those that were there before
-BESIDE = {"girelix": ("digasun",), "bitonex": ("girelix", "fuvirax")}
+BESIDE = {"girelix": ("digasun",), "bitonex": ("girelix", "fuvirax"), "belelorn": ("girelix",)}
 
 
 def mixer_rates(engine, batch, context, prefill_tokens):
@@ -423,6 +441,8 @@ def mixer_rates(engine, batch, context, prefill_tokens):
             mid, mix = m.project(x), m.scan
         elif kind == "LightningAttention":
             mid, mix = m.project(x), m.scan
+        elif kind == "MLSTM":
+            mid, mix = m.project(x, step), m.scan
         else:
             return
         mix(mid, step, v)          # once outside the recording
@@ -448,7 +468,7 @@ def mixer_rates(engine, batch, context, prefill_tokens):
         kv = [v for v in views if isinstance(v, KVView)]
         if kv:
             n = kv[0].need
-            keys = min(context, n.window) if n.window > 0 else context
+            keys = min(context, n.window + n.keep_first) if n.window > 0 else context
             return batch * keys * (n.n_kv_heads * n.head_dim + n.v_heads * n.v_dim) * kv[0].k.element_size()
         return 2 * batch * max(v.tensor[0].numel() * v.tensor.element_size() for v in views)
 
@@ -474,7 +494,7 @@ def mixer_rates(engine, batch, context, prefill_tokens):
 
 
 def run_design(args):
-    """--design fuvirax | digasun | girelix | bitonex: prompt and decode throughput of the design at sizes that resemble a real
+    """--design fuvirax | digasun | girelix | bitonex | belelorn: prompt and decode throughput of the design at sizes that resemble a real
     model's layers (random weights), beside the Llama of equal size (and, for a design that has one, the closest earlier
     design), and the mixing kernels of all alone against their limits."""
     import torch
@@ -577,7 +597,7 @@ def main():
                          "launched kernel by kernel on a cache that is filled without a prompt step; prints its time and "
                          "no JSON line, and says on stderr where it is")
     ap.add_argument("--design", default=None, metavar="NAME",
-                    help="instead of the default measurement: prompt and decode throughput of a design (fuvirax, digasun, girelix, bitonex) at model-like "
+                    help="instead of the default measurement: prompt and decode throughput of a design (fuvirax, digasun, girelix, bitonex, belelorn) at model-like "
                          "layer sizes beside the Llama of equal size, with the mixing kernels alone (--layers, default 6; "
                          "--sizes 1b-like,3b-like)")
     ap.add_argument("--sizes", default=None, help="with --design: which of its sizes, with commas between them")

@@ -66,16 +66,22 @@ class MLSTM(Mixer):
         return 5 * self.H * self.dk * (self.dv + 1) * new
 
     def forward(self, x, step, view):
+        return self.output(self.scan(self.project(x, step), step, view))
+
+    def project(self, x, step):
+        """(rows [q | k | v | g], gate logits float32, whether the step runs in chunks)."""
         rt = self.rt
-        T = x.shape[0]
-        chunks = self.in_chunks and step.max_new >= self.CHUNKS_FROM and T > 4 * step.n_seqs
-        if chunks:
-            proj, logits = rt.linear(x, self.w_rows), rt.linear(x, self.w_gates, out_dtype=torch.float32)
-        else:
-            both = rt.linear(x, self.w_in, out_dtype=torch.float32)
-            proj, logits = both, both[:, self.gates_at:]
-        out = torch.empty(T, self.H * self.dv, dtype=rt.dtype, device=x.device)
-        state = tuple(v.tensor for v in view)
-        rt.ops.matrix_memory(proj, logits, self.bias_i, self.bias_f, self.cap, self.q_scale, self.norm_w, self.eps, state, out, step,
-                             self.H, self.dk, self.dv, chunks)
-        return rt.linear(out, self.w_o, partials=True)
+        if self.in_chunks and step.max_new >= self.CHUNKS_FROM and x.shape[0] > 4 * step.n_seqs:
+            return rt.linear(x, self.w_rows), rt.linear(x, self.w_gates, out_dtype=torch.float32), True
+        both = rt.linear(x, self.w_in, out_dtype=torch.float32)
+        return both, both[:, self.gates_at:], False
+
+    def scan(self, projected, step, view):
+        """The recurrence over the step's tokens, each sequence from its own state -> [tokens, heads * vdim]."""
+        proj, logits, chunks = projected
+        out = torch.empty(proj.shape[0], self.H * self.dv, dtype=self.rt.dtype, device=proj.device)
+        return self.rt.ops.matrix_memory(proj, logits, self.bias_i, self.bias_f, self.cap, self.q_scale, self.norm_w, self.eps,
+                                         tuple(v.tensor for v in view), out, step, self.H, self.dk, self.dv, chunks)
+
+    def output(self, mixed):
+        return self.rt.linear(mixed, self.w_o, partials=True)
