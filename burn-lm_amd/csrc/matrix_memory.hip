@@ -19,8 +19,8 @@
 //   o_t = (sum_s A_ts v_s + c_t S_in^T q_t) / (max(|sum_s A_ts + c_t n_in . q_t|, exp(-m_t)) + 1e-6)
 //   S_out = c_n S_in + sum_s exp(F_n - F_s + i_s - m_n) k_s v_s^T,  n_out likewise
 // All exponents are at most zero.  F is double: a head that forgets fast reaches sums of several hundred within a chunk,
-// and the difference of two of them is the logarithm of a weight.  Kernels: mm_gates (a wavefront per (sequence, head) walks the chunks: prefix sums
-// and prefix maxima over the 64 lanes), mm_state (each chunk's own share of S and n), mm_carry (the chunks' start
+// and the difference of two of them is the logarithm of a weight.  Kernels: mm_gates (a block per (sequence, head), a wavefront per chunk: prefix sums
+// and prefix maxima over the 64 lanes, then m from chunk to chunk), mm_state (each chunk's own share of S and n), mm_carry (the chunks' start
 // states in order), mm_out, then the norm.  Matrix instruction layouts as for lightning attention (recurrent.hip).
 #include "chunk_form.h"
 
@@ -68,7 +68,22 @@ __global__ void __launch_bounds__(256)
   float m = m_state[(size_t)slot * H + h];
   for (int i = tid; i < dk; i += 256) n_sm[i] = nh[i];
   const float bi = bias_i[h], bf = bias_f[h], inv_cap = 1.0f / cap;
+  float s[MM_ROWS][4];
+  auto load_rows = [&](int r0) {
+#pragma unroll
+    for (int u = 0; u < MM_ROWS; ++u) {
+      const int r = r0 + 16 * u;
+      if (VEC) {
+        const float4 x = (r < dk && col < dv) ? *reinterpret_cast<const float4*>(Sh + (size_t)r * dv + col) : make_float4(0.f, 0.f, 0.f, 0.f);
+        s[u][0] = x.x; s[u][1] = x.y; s[u][2] = x.z; s[u][3] = x.w;
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) s[u][e] = (r < dk && col + e < dv) ? Sh[(size_t)r * dv + col + e] : 0.f;
+      }
+    }
+  };
   for (int t = t0; t < t1; ++t) {
+    load_rows(rg);      // the first rows travel while the gates and the denominator are formed
     const TP* row = proj + (size_t)t * ld;
     const MmGates g = mm_gates(z[(size_t)t * ldz + h] + bi, z[(size_t)t * ldz + H + h] + bf, cap, inv_cap);
     const float m_new = fmaxf(g.log_f + m, g.log_i);
@@ -89,18 +104,7 @@ __global__ void __launch_bounds__(256)
     nq = block_sum<true>(nq, red);      // its barrier also hands q and k over (four wavefronts)
     float o[4] = {0.f, 0.f, 0.f, 0.f};
     for (int r0 = rg; r0 < dk; r0 += 16 * MM_ROWS) {
-      float s[MM_ROWS][4];
-#pragma unroll
-      for (int u = 0; u < MM_ROWS; ++u) {
-        const int r = r0 + 16 * u;
-        if (VEC) {
-          const float4 x = (r < dk && col < dv) ? *reinterpret_cast<const float4*>(Sh + (size_t)r * dv + col) : make_float4(0.f, 0.f, 0.f, 0.f);
-          s[u][0] = x.x; s[u][1] = x.y; s[u][2] = x.z; s[u][3] = x.w;
-        } else {
-#pragma unroll
-          for (int e = 0; e < 4; ++e) s[u][e] = (r < dk && col + e < dv) ? Sh[(size_t)r * dv + col + e] : 0.f;
-        }
-      }
+      if (r0 != rg) load_rows(r0);
 #pragma unroll
       for (int u = 0; u < MM_ROWS; ++u) {
         const int r = r0 + 16 * u;
@@ -186,28 +190,24 @@ extern "C" int blm_mm_step(const void* proj, int proj_dtype, int ld, const float
 // ---- prompts ------------------------------------------------------------------------------------------
 // sums [H][T] double: F (the chunk's running sum of log f); gates [2][H][T] float: log i, m; chunk [B][n_seg][H][2] float: m at the chunk's
 // start, and c_n, what the chunk leaves of its start state.  Leaves the sequence's m.
-__global__ void __launch_bounds__(BLM_WAVE)
+#define MM_GATE_WAVES 16
+__global__ void __launch_bounds__(MM_GATE_WAVES* BLM_WAVE)
     mm_gates_kernel(const float* __restrict__ z, int ldz, const float* __restrict__ bias_i, const float* __restrict__ bias_f,
                     float cap, double* __restrict__ sums, float* __restrict__ gates, float* __restrict__ chunk,
                     float* __restrict__ m_state,
                     const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slots, int T, int H, int n_seg) {
-  const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x;
+  __shared__ double F_end[MM_GATE_WAVES], top_end[MM_GATE_WAVES];
+  __shared__ float m_at[MM_GATE_WAVES + 1];      // m at the start of each wavefront's chunk, and behind the last one
+  const int h = blockIdx.x, b = blockIdx.y, wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
   const int slot = seq_slots[b], first = cu_seqlens[b], n_new = cu_seqlens[b + 1] - first;
   if (slot < 0 || n_new <= 0) return;
-  float m_in = m_state[(size_t)slot * H + h];
+  if (threadIdx.x == 0) m_at[MM_GATE_WAVES] = m_state[(size_t)slot * H + h];
   const float bi = bias_i[h], bf = bias_f[h], inv_cap = 1.0f / cap;
-  float zi = 0.f, zf = 0.f;
-  auto fetch = [&](int t) {
-    if (t < n_new) {
-      zi = z[(size_t)(first + t) * ldz + h];
-      zf = z[(size_t)(first + t) * ldz + H + h];
-    }
-  };
-  fetch(lane);
-  for (int c = 0, t0 = 0; t0 < n_new; ++c, t0 += LC_CHUNK) {
-    const bool valid = t0 + lane < n_new;
-    const MmGates g = mm_gates(zi + bi, zf + bf, cap, inv_cap);
-    fetch(t0 + LC_CHUNK + lane);      // the next chunk's logits travel meanwhile
+  for (int base = 0; base < n_new; base += MM_GATE_WAVES * LC_CHUNK) {      // sixteen chunks at a time
+    const int t0 = base + wave * LC_CHUNK, t = t0 + lane;
+    const bool valid = t < n_new;
+    const float* row = z + (size_t)(first + min(t, n_new - 1)) * ldz;
+    const MmGates g = mm_gates(row[h] + bi, row[H + h] + bf, cap, inv_cap);
     double F = valid ? (double)g.log_f : 0.0;
 #pragma unroll
     for (int d = 1; d < BLM_WAVE; d <<= 1) {
@@ -220,24 +220,36 @@ __global__ void __launch_bounds__(BLM_WAVE)
       const double o = __shfl_up(top, d, BLM_WAVE);
       if (lane >= d) top = fmax(top, o);
     }
-    const float m = (float)(F + fmax((double)m_in, top));
-    if (valid) {
-      const size_t at = (size_t)h * T + first + t0 + lane;
-      sums[at] = F;
-      gates[at] = g.log_i;
-      gates[(size_t)H * T + at] = m;
+    // lanes behind the sequence add nothing to either: the last lane holds the chunk's sum and maximum
+    if (lane == BLM_WAVE - 1) { F_end[wave] = F; top_end[wave] = top; }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+      float m = m_at[MM_GATE_WAVES];
+      for (int w = 0; w < MM_GATE_WAVES; ++w) {
+        m_at[w] = m;
+        if (base + w * LC_CHUNK < n_new) m = (float)(F_end[w] + fmax((double)m, top_end[w]));
+      }
+      m_at[MM_GATE_WAVES] = m;
     }
-    const int last = min(n_new - t0, LC_CHUNK) - 1;
-    const double F_n = __shfl(F, last, BLM_WAVE);
-    const float m_n = __shfl(m, last, BLM_WAVE);
-    if (lane == 0) {
-      float* ck = chunk + (((size_t)b * n_seg + c) * H + h) * 2;
-      ck[0] = m_in;
-      ck[1] = expf((float)(F_n + (double)m_in - (double)m_n));
+    __syncthreads();
+    if (t0 < n_new) {
+      const float m_in = m_at[wave];
+      const float m = (float)(F + fmax((double)m_in, top));
+      if (valid) {
+        const size_t at = (size_t)h * T + first + t;
+        sums[at] = F;
+        gates[at] = g.log_i;
+        gates[(size_t)H * T + at] = m;
+      }
+      if (lane == BLM_WAVE - 1) {      // its F and m are the chunk's last token's
+        float* ck = chunk + (((size_t)b * n_seg + t0 / LC_CHUNK) * H + h) * 2;
+        ck[0] = m_in;
+        ck[1] = expf((float)(F + (double)m_in - (double)m));
+      }
     }
-    m_in = m_n;
+    __syncthreads();      // the next sixteen chunks write the same places
   }
-  if (lane == 0) m_state[(size_t)slot * H + h] = m_in;
+  if (threadIdx.x == 0) m_state[(size_t)slot * H + h] = m_at[MM_GATE_WAVES];
 }
 
 // seg_end [B][n_seg][H][dk][dv], seg_n [B][n_seg][H][dk]: what the chunk's own tokens add to S and n by the chunk's end
@@ -562,7 +574,7 @@ extern "C" int blm_mm_chunks(const void* proj, int dtype, int ld, const float* z
   int dev = -1;
   BLM_REQUIRE(hipGetDevice(&dev) == hipSuccess && dev >= 0 && dev < MM_DEVICES && g_mm_ready[dev],
               "mm_chunks: blm_mm_chunks_init has not run on device %d", dev);
-  hipLaunchKernelGGL(mm_gates_kernel, dim3(H, B), dim3(BLM_WAVE), 0, stream, z, ldz, bias_i, bias_f, cap, sums, gates, chunk, m_state,
+  hipLaunchKernelGGL(mm_gates_kernel, dim3(H, B), dim3(MM_GATE_WAVES * BLM_WAVE), 0, stream, z, ldz, bias_i, bias_f, cap, sums, gates, chunk, m_state,
                      cu_seqlens, seq_slots, T, H, n_seg);
   BLM_LAUNCH_CHECK("mm_gates");
   const dim3 grid((unsigned)n_seg, (unsigned)(H * n_vt), (unsigned)B);

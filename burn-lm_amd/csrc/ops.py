@@ -10,7 +10,7 @@ import torch
 
 from . import build as _build
 
-ABI_VERSION = 39
+ABI_VERSION = 40
 _lib = None
 _lock = threading.Lock()
 
@@ -62,6 +62,7 @@ _SIGNATURES = {
     "blm_post_norm": [_c_void_p] + [_c_void_p, _c_int, _c_int, ctypes.c_longlong, _c_float, _c_void_p, _c_float] * 2
                      + [_c_void_p, _c_float, _c_int, _c_void_p, _c_int, _c_void_p, _c_float, _c_void_p, _c_int, _c_int, _c_void_p,
                         _c_int, _c_int, _c_void_p],
+    "blm_sum_planes": [_c_void_p, _c_int, ctypes.c_longlong, _c_void_p, _c_void_p],
     "blm_embed_positions": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int,
                             _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "blm_mm_step": [_c_void_p, _c_int, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_float, _c_float, _c_void_p, _c_float,
@@ -1380,6 +1381,14 @@ def post_norm(h, terms, post=None, fresh=False, vec=None, write_h=True, gamma=No
     _call("blm_post_norm", h.data_ptr(), *args, _ptr(post[0]) if post else 0, float(post[1]) if post else 0.0, 1 if fresh else 0,
           _ptr(vec), 1 if write_h else 0, _ptr(gamma), float(eps), _ptr(out), _code(out) if out is not None else 0,
           out.stride(0) if out is not None else 0, _ptr(rows), n, D, _stream())
+    return out
+
+
+def sum_planes(planes, out):
+    """out = the sum of planes float32 [P, M, N] over P, in order."""
+    _gpu(planes, out)
+    _f32("planes", planes); _f32("out", out, planes[0].numel())
+    _call("blm_sum_planes", planes.data_ptr(), planes.shape[0], out.numel(), out.data_ptr(), _stream())
     return out
 
 

@@ -323,3 +323,30 @@ extern "C" int blm_embed_positions(const void* table, int table_dtype, const int
   BLM_LAUNCH_CHECK("embed_positions");
   return 0;
 }
+
+// ---------------------------------------------------------------------------------------
+// out[e] = sum over planes p of y[p][e], in order, float: the partial products of a narrow matrix product
+// ---------------------------------------------------------------------------------------
+__global__ void sum_planes_kernel(const float* __restrict__ y, int planes, long long n, float* __restrict__ out) {
+  const long long stride = (long long)gridDim.x * blockDim.x;
+  for (long long e = (long long)blockIdx.x * blockDim.x + threadIdx.x; e < n; e += stride) {
+    float v = 0.f;
+    for (int p0 = 0; p0 < planes; p0 += 8) {
+      float a[8];
+#pragma unroll
+      for (int q = 0; q < 8; ++q) a[q] = y[(size_t)min(p0 + q, planes - 1) * n + e];
+#pragma unroll
+      for (int q = 0; q < 8; ++q)
+        if (p0 + q < planes) v += a[q];
+    }
+    out[e] = v;
+  }
+}
+
+extern "C" int blm_sum_planes(const float* y, int planes, long long n, float* out, hipStream_t stream) {
+  BLM_REQUIRE(planes >= 1 && n > 0, "sum_planes: bad sizes, %d planes", planes);
+  const unsigned blocks = (unsigned)((n + 255) / 256 < 65535 ? (n + 255) / 256 : 65535);
+  hipLaunchKernelGGL(sum_planes_kernel, dim3(blocks), dim3(256), 0, stream, y, planes, n, out);
+  BLM_LAUNCH_CHECK("sum_planes");
+  return 0;
+}

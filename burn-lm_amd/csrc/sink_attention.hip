@@ -97,6 +97,59 @@ __global__ void qkv_prepare_kernel(TA* __restrict__ qkv, int ld, const float* __
   }
 }
 
+// The same for unit-norm heads that do not turn: a wavefront per head, whose lanes stay in registers between the norm and
+// the stores (dk up to 64 * QU_LANES).  grid (tokens, blocks of four heads: H queries, then G keys, then, where the values
+// have columns of their own, G values)
+#define QU_LANES 8
+template <typename TA>
+__global__ void __launch_bounds__(256)
+    qkv_unit_kernel(TA* __restrict__ qkv, int ld, const float* __restrict__ bias, const int* __restrict__ positions,
+                    const int* __restrict__ token_seq, const int* __restrict__ block_table, int table_width, TA* __restrict__ kcache,
+                    TA* __restrict__ vcache, int page_size, int H, int G, int dk, int dv, int n_heads, int values_are_keys,
+                    const float* __restrict__ q_scale, float norm_eps) {
+  const int t = blockIdx.x, lane = threadIdx.x & (BLM_WAVE - 1);
+  const int head = blockIdx.y * 4 + threadIdx.x / BLM_WAVE;
+  if (head >= n_heads) return;
+  const int b = token_seq[t];
+  if (b < 0) return;
+  TA* row = qkv + (size_t)t * ld;
+  const bool value = head >= H + G;
+  const int col = value ? (H + G) * dk + (head - H - G) * dv : head * dk, n = value ? dv : dk;
+  const int pos = positions[t];
+  size_t page = 0;
+  if (head >= H) page = block_table[(size_t)b * table_width + pos / page_size];
+  const int in_page = pos % page_size;
+  float x[QU_LANES];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < QU_LANES; ++k) {
+    const int d = lane + k * BLM_WAVE;
+    x[k] = d < n ? to_float(row[col + d]) + (bias ? bias[col + d] : 0.f) : 0.f;
+    ss = fmaf(x[k], x[k], ss);
+  }
+  const float f = value ? 1.0f : 1.0f / sqrtf(wave_sum(ss) / (float)dk + norm_eps);
+  if (head < H) {
+    const float fq = f * (q_scale ? q_scale[head] : 1.0f);
+#pragma unroll
+    for (int k = 0; k < QU_LANES; ++k) {
+      const int d = lane + k * BLM_WAVE;
+      if (d < n) row[col + d] = from_float<TA>(x[k] * fq);
+    }
+    return;
+  }
+  const int c = value ? head - H - G : head - H;
+  TA* krow = kcache + ((page * G + c) * page_size + in_page) * dk;
+  TA* vcol = vcache + (page * G + c) * (size_t)dv * page_size + in_page;
+#pragma unroll
+  for (int k = 0; k < QU_LANES; ++k) {
+    const int d = lane + k * BLM_WAVE;
+    if (d < n) {
+      if (!value) krow[d] = from_float<TA>(x[k] * f);
+      if (value || values_are_keys) vcol[(size_t)d * page_size] = from_float<TA>(x[k]);
+    }
+  }
+}
+
 extern "C" int blm_qkv_prepare(void* qkv, int dtype, int ld, const float* bias, const float* cos_sin, int rot,
                                const int* positions, const int* token_seq, const int* block_table, int table_width,
                                void* kcache, void* vcache, int page_size, int T, int H, int G, int dk, int dv, int write_kv,
@@ -110,6 +163,18 @@ extern "C" int blm_qkv_prepare(void* qkv, int dtype, int ld, const float* bias, 
   BLM_REQUIRE(rot == 0 || cos_sin, "qkv_prepare: the table of angles is missing");
   const size_t factors = unit_norm ? (size_t)(H + G) * sizeof(float) : 0;
   BLM_REQUIRE(factors <= 60 * 1024, "qkv_prepare: %d heads are too many", H + G);
+  if (unit_norm && rot == 0 && dk <= BLM_WAVE * QU_LANES && dv <= BLM_WAVE * QU_LANES && (dtype == BLM_F32 || dtype == BLM_BF16)) {
+    const int n_heads = H + (write_kv ? G + (values_are_keys ? 0 : G) : 0);
+    const dim3 grid(T, (n_heads + 3) / 4);
+    if (dtype == BLM_F32)
+      hipLaunchKernelGGL(qkv_unit_kernel<float>, grid, dim3(256), 0, stream, (float*)qkv, ld, bias, positions, token_seq, block_table,
+                         table_width, (float*)kcache, (float*)vcache, page_size, H, G, dk, dv, n_heads, values_are_keys, q_scale, norm_eps);
+    else
+      hipLaunchKernelGGL(qkv_unit_kernel<bf16>, grid, dim3(256), 0, stream, (bf16*)qkv, ld, bias, positions, token_seq, block_table,
+                         table_width, (bf16*)kcache, (bf16*)vcache, page_size, H, G, dk, dv, n_heads, values_are_keys, q_scale, norm_eps);
+    BLM_LAUNCH_CHECK("qkv_unit");
+    return 0;
+  }
   if (dtype == BLM_F32)
     hipLaunchKernelGGL(qkv_prepare_kernel<float>, dim3(T), dim3(256), factors, stream, (float*)qkv, ld, bias, cos_sin, rot, positions,
                        token_seq, block_table, table_width, (float*)kcache, (float*)vcache, page_size, H, G, dk, dv, write_kv, adjacent, values_are_keys, q_scale, unit_norm, norm_eps);

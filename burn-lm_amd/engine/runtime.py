@@ -58,6 +58,7 @@ RING_QKV_K = 6144
 # over whole prompts, 2-5 % faster up to 512 tokens and equal beyond).
 MFMA_MIN_GROUP_K = 768
 MID_PLANES_MAX_ROWS = 512
+NARROW_MIN_GROUP_K = 256
 # Rows for which the fused gate/up product is used when it is switched on (below, the library is
 # ahead by far; above, its better rate on long runs of tiles has made up for the extra pass).
 FUSED_GATE_UP_ROWS = (192, 4096)
@@ -285,6 +286,17 @@ class Runtime:
                     best = (g, tile, blocks)
         return best[0], best[1]
 
+    def narrow_groups(self, M, N, K):
+        """Groups of K for a float32 result of at most 64 columns and many rows (a router's logits, the gates of a
+        recurrence): its row tiles alone are a handful of blocks, each walking all of K; cut into groups of at least
+        NARROW_MIN_GROUP_K the product fills the chip, and a small kernel adds the planes.  1: not worth it."""
+        if N > 64 or M <= MFMA_SKINNY_MAX_ROWS:
+            return 1
+        tiles, groups = -(-M // 128), 1
+        while groups < 16 and K // (groups * 2) >= NARROW_MIN_GROUP_K and tiles * groups * 2 <= self.compute_units:
+            groups *= 2
+        return groups
+
     def mid_k_groups(self, M, N, K):
         """Groups of K of mid_planes_plan (0: the library's product)."""
         return self.mid_planes_plan(M, N, K)[0]
@@ -353,6 +365,15 @@ class Runtime:
             out = torch.empty(M, N, dtype=out_dtype, device=x.device)
         if (out_dtype == torch.float32 and M > 32 and aligned and x.dtype == w.dtype == torch.bfloat16
                 and x.stride(1) == 1 and w.is_contiguous() and out.stride(1) == 1 and N * K * 2 < 1 << 32):
+            groups = self.narrow_groups(M, N, K) if out.is_contiguous() else 1
+            if groups > 1:
+                planes = torch.empty(groups, M, N, dtype=torch.float32, device=x.device)
+                return ops.sum_planes(ops.gemm_mfma(x, w, planes, tile=(128, 64, 6)), out)
+            tiles = -(-M // 256) * -(-N // 128)
+            if planes and M > MID_PLANES_MAX_ROWS and tiles * 2 <= self.compute_units and K >= 2 * MFMA_MIN_GROUP_K:
+                # a residual's new start: partial planes fill the chip where the tiles alone leave half of it idle, and
+                # the norm behind it adds them (2,048 rows, width 2048, K = 4096: 42.4 us against 57.9)
+                return ops.gemm_mfma(x, w, torch.empty(2, M, N, dtype=torch.float32, device=x.device), tile=(256, 128))
             # float32 results (logits) for more rows than one skinny product takes at this width (more than 64,
             # or more than 32 where K is above 2048): the matrix-core kernel with a float output, which reads
             # the weights once.  Measured per call with a vocabulary of 128,256 against the skinny product in

@@ -529,6 +529,49 @@ def test_drawn_configurations(tmp_path, seed, dtype):
     rows.check()
 
 
+@pytest.mark.gpu
+def test_a_middle_sized_model_in_bfloat16(tmp_path):
+    """Sizes at which products run on the matrix cores in every form: a prompt of more than 512 tokens (the loop's entry as
+    partial planes, routers and gates in groups of K), decode steps of one, 20 and 70 sequences."""
+    cfg = config([pair(heads=8, kv_heads=2, dim=64, scale=0.125, size=200, keep=5, r_heads=4, r_dim=64, r_vdim=96, decay=(0.5, 0.9, 0.99, 1.0),
+                       mlp=dense(1024)),
+                  memory(heads=4, dim=64, vdim=128, mlp=moe(experts=8, top=2, ff=64, shared=128))], width=768, vocab=512, loop=(0, 2, 2))
+    w = make_weights(cfg, 14)
+    eng = engine_for(tmp_path, cfg, w, "bfloat16", max_tokens=8192, max_seqs=72)
+    long = tokens_of(cfg, 70, 603)
+    want = P.forward(w, cfg, long)
+    rows = Rows("bfloat16")
+    s = eng.open()
+    rows.add(eng.step([(s, long[:600], list(range(600)))]).double().cpu().numpy(), want[:600], "prompt")
+    for k in range(600, 603):
+        rows.add(eng.step([(s, [long[k]], [0])]).double().cpu().numpy(), want[k:k + 1], k)
+    eng.close(s)
+    short = [tokens_of(cfg, 80 + i, 12) for i in range(4)]
+    wants = [P.forward(w, cfg, t) for t in short]
+    for n in (20, 70):
+        slots = [eng.open() for _ in range(n)]
+        got = eng.step([(s, short[i % 4][:9], [8]) for i, s in enumerate(slots)]).double().cpu().numpy()
+        rows.add(got, np.stack([wants[i % 4][8] for i in range(n)]), n)
+        for k in (9, 10, 11):
+            got = eng.step([(s, [short[i % 4][k]], [0]) for i, s in enumerate(slots)]).double().cpu().numpy()
+            rows.add(got, np.stack([wants[i % 4][k] for i in range(n)]), (n, k))
+        for s in slots:
+            eng.close(s)
+    rows.check()
+
+
+@pytest.mark.gpu
+def test_narrow_float_products_in_groups():
+    from burn_lm_amd.engine.runtime import Runtime
+    rt = Runtime()
+    g = torch.Generator().manual_seed(0)
+    for M, N, K in ((300, 16, 2048), (65, 8, 512), (130, 64, 1536), (2000, 48, 768), (300, 72, 2048)):
+        x, w = (torch.randn(n, K, generator=g).to("cuda", torch.bfloat16) for n in (M, N))
+        assert (rt.narrow_groups(M, N, K) > 1) == (N <= 64)
+        want = (x.double() @ w.double().t()).cpu().numpy()
+        assert rel_err(rt.linear(x, rt.weight(w), out_dtype=torch.float32).double().cpu().numpy(), want) < 1e-5, (M, N, K)
+
+
 class _Step:
     """The index arrays that the kernels read, for sequences laid out by hand; `padding` tokens of no sequence behind."""
 
