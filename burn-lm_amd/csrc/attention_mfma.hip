@@ -47,6 +47,12 @@ __device__ __forceinline__ float coherent_load(const float* p) {
   return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
 }
 
+// a result in bfloat16 or, out_f32, as it is
+__device__ __forceinline__ void am_store(void* out, size_t at, float v, int out_f32) {
+  if (out_f32) static_cast<float*>(out)[at] = v;
+  else static_cast<bf16*>(out)[at] = from_float<bf16>(v);
+}
+
 // keep the first n (0..4) bf16 of an 8-byte group, zero the rest
 __device__ __forceinline__ uint2 keep_first(uint2 v, int n) {
   if (n >= 4) return v;
@@ -337,11 +343,11 @@ __device__ __forceinline__ void load_q(const bf16* qrow, uint4* qf) {
 // ---------------------------------------------------------------------------------------
 template <int HD, bool EXT>
 __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 4 : (HD <= 128 ? 2 : 1), HD <= 64 ? 8 : (HD <= 128 ? 2 : 1))))
-    attn_prefill_mfma_kernel(const bf16* __restrict__ q, int q_row_stride, bf16* __restrict__ out,
+    attn_prefill_mfma_kernel(const bf16* __restrict__ q, int q_row_stride, void* __restrict__ out,
                              const int* __restrict__ positions, const int* __restrict__ cu_seqlens,
                              const int* __restrict__ block_table, int table_width,
                              const bf16* __restrict__ kcache, const bf16* __restrict__ vcache, int nh, int nkv,
-                             float scale, int window, const float* __restrict__ sinks, int keep_first, float cap) {
+                             float scale, int window, const float* __restrict__ sinks, int keep_first, float cap, int out_f32) {
   constexpr int KS = (HD + 31) / 32;
   constexpr int DT = (HD + 15) / 16;
   // Head sizes 64 and 128: a page comes straight from global memory into shared memory, its rows'
@@ -494,11 +500,15 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
   const float l = lsum[0];
   if (c < nq) {
     const float inv = 1.0f / l;
-    bf16* orow = out + (size_t)row * nh * HD + (size_t)head * HD;
+    const size_t at = (size_t)row * nh * HD + (size_t)head * HD;
+    bf16* orow = static_cast<bf16*>(out) + at;
+    float* frow = static_cast<float*>(out) + at;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       const int d = dt * 16 + kg * 4;
-      if (HD % 16 == 0 || d < HD) {
+      if (out_f32) {
+        *reinterpret_cast<float4*>(frow + d) = make_float4(o[dt][0] * inv, o[dt][1] * inv, o[dt][2] * inv, o[dt][3] * inv);
+      } else if (HD % 16 == 0 || d < HD) {
         uint2 w;
         w.x = pack_bf16x2(o[dt][0] * inv, o[dt][1] * inv);
         w.y = pack_bf16x2(o[dt][2] * inv, o[dt][3] * inv);
@@ -641,11 +651,11 @@ __device__ __forceinline__ void attn_page32(const bf16* __restrict__ kp, const b
 // of the 16-query kernel above
 template <int HD, bool EXT>
 __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 4 : 2, HD <= 64 ? 4 : 2)))
-    attn_prefill32_kernel(const bf16* __restrict__ q, int q_row_stride, bf16* __restrict__ out,
+    attn_prefill32_kernel(const bf16* __restrict__ q, int q_row_stride, void* __restrict__ out,
                           const int* __restrict__ positions, const int* __restrict__ cu_seqlens,
                           const int* __restrict__ block_table, int table_width,
                           const bf16* __restrict__ kcache, const bf16* __restrict__ vcache, int nh, int nkv,
-                          float scale, int window, const float* __restrict__ sinks, int keep_first, float cap) {
+                          float scale, int window, const float* __restrict__ sinks, int keep_first, float cap, int out_f32) {
   static_assert(HD % 32 == 0 && HD <= 128, "32-query prefill: head sizes 32, 64, 96, 128");
   constexpr int KS = HD / 16, RT = HD / 32, QT = 32;
   constexpr bool DIRECT = HD == 64 || HD == 128;   // as in the 16-query kernel
@@ -779,11 +789,18 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE) __attribute__((amdgpu_wave
   }
   if (!active || j >= nq) return;
   const float inv = 1.0f / lsum;
-  bf16* orow = out + (size_t)row * nh * HD + (size_t)head * HD;
+  const size_t at = (size_t)row * nh * HD + (size_t)head * HD;
+  bf16* orow = static_cast<bf16*>(out) + at;
+  float* frow = static_cast<float*>(out) + at;
 #pragma unroll
   for (int rt = 0; rt < RT; ++rt)
 #pragma unroll
     for (int gq = 0; gq < 4; ++gq) {   // four neighbouring dims per store: rt * 32 + 8 gq + 4 hb ..
+      if (out_f32) {
+        *reinterpret_cast<float4*>(frow + rt * 32 + 8 * gq + 4 * hb) =
+            make_float4(o[rt][4 * gq + 0] * inv, o[rt][4 * gq + 1] * inv, o[rt][4 * gq + 2] * inv, o[rt][4 * gq + 3] * inv);
+        continue;
+      }
       uint2 w;
       w.x = pack_bf16x2(o[rt][4 * gq + 0] * inv, o[rt][4 * gq + 1] * inv);
       w.y = pack_bf16x2(o[rt][4 * gq + 2] * inv, o[rt][4 * gq + 3] * inv);
@@ -804,8 +821,8 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE)
                             const int* __restrict__ token_seq, const int* __restrict__ block_table,
                             int table_width, const bf16* __restrict__ kcache, const bf16* __restrict__ vcache,
                             int nh, int nkv, float scale, int window, int n_splits, float* part_o,
-                            float* part_ml, int* arrivals, bf16* out, const float* __restrict__ sinks, int keep_first,
-                            float cap) {
+                            float* part_ml, int* arrivals, void* out, const float* __restrict__ sinks, int keep_first,
+                            float cap, int out_f32) {
   constexpr int KS = (HD + 31) / 32;
   constexpr int DT = (HD + 15) / 16;
   // Every wavefront brings its pages through a staging area of its own in shared memory: whole
@@ -916,7 +933,7 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE)
       O += reinterpret_cast<const float*>(sm_area[k])[cc * HD + d] * f;
     }
     if (n_splits == 1 || b < 0) {   // nothing to merge (a padding token gives zeros)
-      out[((size_t)t * nh + kvh * G + g0 + cc) * HD + d] = from_float<bf16>(b < 0 ? 0.f : O / L);
+      am_store(out, ((size_t)t * nh + kvh * G + g0 + cc) * HD + d, b < 0 ? 0.f : O / L, out_f32);
     } else {
       const size_t at = ((size_t)t * nh + kvh * G + g0 + cc) * n_splits + split;
       coherent_store(part_o + at * HD + d, O);
@@ -977,7 +994,7 @@ __global__ void __launch_bounds__(AM_WAVES* BLM_WAVE)
       }
       M = Mc;
     }
-    out[head_at * HD + d] = from_float<bf16>(O / L);
+    am_store(out, head_at * HD + d, O / L, out_f32);
   }
 }
 
@@ -1004,7 +1021,7 @@ extern "C" int blm_attn_prefill_mfma(const void* q, int q_row_stride, void* out,
                                      const int* positions, const int* cu_seqlens, const int* block_table,
                                      int table_width, const void* kcache, const void* vcache, int page_size,
                                      int n_seqs, int max_new, int nh, int nkv, int hd, float scale, int window,
-                                     int queries, const float* sinks, int keep_first, float cap, hipStream_t stream) {
+                                     int queries, const float* sinks, int keep_first, float cap, int out_f32, hipStream_t stream) {
   BLM_REQUIRE(n_seqs > 0 && n_seqs <= 65535 && max_new > 0 && nh > 0 && nkv > 0 && nkv <= 65535 && nh % nkv == 0,
               "attn_prefill_mfma: bad sizes seqs=%d max_new=%d heads=%d kv_heads=%d", n_seqs, max_new, nh, nkv);
   BLM_REQUIRE(blm_attn_prefill_mfma_supported(act_dtype, hd, page_size),
@@ -1033,12 +1050,12 @@ extern "C" int blm_attn_prefill_mfma(const void* q, int q_row_stride, void* out,
   case HD:                                                                                                       \
     if (extended)                                                                                                \
       hipLaunchKernelGGL((attn_prefill32_kernel<HD, true>), grid32, block32, 0, stream, (const bf16*)q, q_row_stride, \
-                         (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
-                         (const bf16*)vcache, nh, nkv, scale, window, sinks, keep_first, cap);                    \
+                         out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
+                         (const bf16*)vcache, nh, nkv, scale, window, sinks, keep_first, cap, out_f32);           \
     else                                                                                                         \
       hipLaunchKernelGGL((attn_prefill32_kernel<HD, false>), grid32, block32, 0, stream, (const bf16*)q, q_row_stride, \
-                         (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
-                         (const bf16*)vcache, nh, nkv, scale, window, sinks, 0, 0.f);                             \
+                         out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
+                         (const bf16*)vcache, nh, nkv, scale, window, sinks, 0, 0.f, out_f32);                    \
     break
     switch (hd) {
       BLM_AP32(32); BLM_AP32(64); BLM_AP32(96); BLM_AP32(128);
@@ -1053,12 +1070,12 @@ extern "C" int blm_attn_prefill_mfma(const void* q, int q_row_stride, void* out,
   case HD:                                                                                                       \
     if (extended)                                                                                                \
       hipLaunchKernelGGL((attn_prefill_mfma_kernel<HD, true>), grid, block, 0, stream, (const bf16*)q, q_row_stride, \
-                         (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
-                         (const bf16*)vcache, nh, nkv, scale, window, sinks, keep_first, cap);                    \
+                         out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
+                         (const bf16*)vcache, nh, nkv, scale, window, sinks, keep_first, cap, out_f32);           \
     else                                                                                                         \
       hipLaunchKernelGGL((attn_prefill_mfma_kernel<HD, false>), grid, block, 0, stream, (const bf16*)q, q_row_stride, \
-                         (bf16*)out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
-                         (const bf16*)vcache, nh, nkv, scale, window, sinks, 0, 0.f);                             \
+                         out, positions, cu_seqlens, block_table, table_width, (const bf16*)kcache,        \
+                         (const bf16*)vcache, nh, nkv, scale, window, sinks, 0, 0.f, out_f32);                    \
     break
   switch (hd) {
     BLM_AP(16); BLM_AP(32); BLM_AP(48); BLM_AP(64); BLM_AP(80); BLM_AP(96); BLM_AP(112); BLM_AP(128); BLM_AP(256);
@@ -1075,7 +1092,7 @@ extern "C" int blm_attn_decode(const void* q, int q_row_stride, void* out, int a
                                const int* token_seq, const int* block_table, int table_width, const void* kcache,
                                const void* vcache, int page_size, int T, int nh, int nkv, int hd, float scale,
                                int window, int n_splits, float* part_o, float* part_ml, int* arrivals,
-                               const float* sinks, int keep_first, float cap, hipStream_t stream) {
+                               const float* sinks, int keep_first, float cap, int out_f32, hipStream_t stream) {
   BLM_REQUIRE(keep_first >= 0 && cap >= 0.f, "attn_decode: keep_first %d or cap %g is negative", keep_first, (double)cap);
   BLM_REQUIRE(T > 0 && T <= 65535 && nh > 0 && nkv > 0 && nh % nkv == 0,
               "attn_decode: bad sizes T=%d heads=%d kv_heads=%d", T, nh, nkv);
@@ -1097,11 +1114,11 @@ extern "C" int blm_attn_decode(const void* q, int q_row_stride, void* out, int a
     if (keep_first > 0 || cap > 0.f)                                                                               \
       hipLaunchKernelGGL((attn_decode_mfma_kernel<HD, true>), grid, block, 0, stream, (const bf16*)q, q_row_stride, \
                          positions, token_seq, block_table, table_width, (const bf16*)kcache, (const bf16*)vcache,  \
-                         nh, nkv, scale, window, n_splits, part_o, part_ml, arrivals, (bf16*)out, sinks, keep_first, cap); \
+                         nh, nkv, scale, window, n_splits, part_o, part_ml, arrivals, out, sinks, keep_first, cap, out_f32); \
     else                                                                                                           \
       hipLaunchKernelGGL((attn_decode_mfma_kernel<HD, false>), grid, block, 0, stream, (const bf16*)q, q_row_stride, \
                          positions, token_seq, block_table, table_width, (const bf16*)kcache, (const bf16*)vcache,  \
-                         nh, nkv, scale, window, n_splits, part_o, part_ml, arrivals, (bf16*)out, sinks, 0, 0.f);   \
+                         nh, nkv, scale, window, n_splits, part_o, part_ml, arrivals, out, sinks, 0, 0.f, out_f32);   \
     break
   switch (hd) { BLM_AD(16); BLM_AD(32); BLM_AD(48); BLM_AD(64); BLM_AD(80); BLM_AD(96); BLM_AD(112); BLM_AD(128); }
 #undef BLM_AD

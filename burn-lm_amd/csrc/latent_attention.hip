@@ -7,6 +7,9 @@
 // R + Dr lanes against the cache row, and a head's result is the probability-weighted sum of latents
 // (R lanes), which the caller expands with W_uv.
 //
+// A window limits how far back a query sees (row j of position p while p - j < window; 0: every earlier row), and a sink,
+// one logit per head (not scaled, without row or value), may take a share of the softmax's denominator.
+//
 // Kernels: the write of a step's tokens into the cache (RMS norm of the latent, rotation of the shared
 // key part and of the queries' rotated parts), a small batched product per head, and the attention.
 #include "common.h"
@@ -237,7 +240,7 @@ extern "C" int blm_head_project(const void* in, int in_dtype, long long in_row, 
 
 // ---------------------------------------------------------------------------------------
 // The attention, generic form: one wavefront per (query token, head); prompts and decoding alike.
-// Query at position p of its sequence sees rows j <= p of the same sequence.  A chunk of 64 rows at a
+// Query at position p of its sequence sees rows j <= p of the same sequence (those of the window).  A chunk of 64 rows at a
 // time: every lane scores one row (R + Dr lanes against the query in shared memory), the running maximum
 // and sum follow, then every lane owns latent lanes lane, lane + 64, ... of the weighted sum and walks the
 // chunk's rows.  With n_splits > 1 the rows of a (token, head) are cut into pieces for different
@@ -251,7 +254,8 @@ __global__ void __launch_bounds__(LAT_WAVES* BLM_WAVE)
     latent_attn_kernel(const float* __restrict__ qabs, float* __restrict__ olat, const int* __restrict__ positions,
                        const int* __restrict__ token_seq, const int* __restrict__ block_table, int table_width,
                        const TA* __restrict__ kcache, int page_size, int T, int H, int R, int Dr, float scale,
-                       int n_splits, float* part_o, float* part_ml, int* arrivals) {
+                       int n_splits, float* part_o, float* part_ml, int* arrivals, int window,
+                       const float* __restrict__ sinks) {
   extern __shared__ float smem[];
   const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
   const int W = R + Dr;
@@ -274,12 +278,14 @@ __global__ void __launch_bounds__(LAT_WAVES* BLM_WAVE)
   const int pos = positions[t];
   const int* bt = block_table + (size_t)b * table_width;
   const int split = blockIdx.y;
-  const int n_chunks = pos / BLM_WAVE + 1;
+  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;      // the first row seen
+  const int n_chunks = (pos - lo) / BLM_WAVE + 1;
   const int per_split = (n_chunks + n_splits - 1) / n_splits;
-  const int j_begin = split * per_split * BLM_WAVE;
+  const int j_begin = lo + split * per_split * BLM_WAVE;
   const int j_end = min(pos, j_begin + per_split * BLM_WAVE - 1);
 
-  float m = -INFINITY, l = 0.f;
+  const bool sunk = sinks != nullptr && split == 0;      // a sink counts once
+  float m = sunk ? sinks[(int)(item - (long long)t * H)] : -INFINITY, l = sunk ? 1.f : 0.f;
   float acc[LAT_MAX_R / BLM_WAVE];
 #pragma unroll
   for (int i = 0; i < LAT_MAX_R / BLM_WAVE; ++i) acc[i] = 0.f;
@@ -389,10 +395,10 @@ __global__ void __launch_bounds__(LAT_WAVES* BLM_WAVE)
 extern "C" int blm_latent_attn(const float* qabs, float* olat, int cache_dtype, const int* positions,
                                const int* token_seq, const int* block_table, int table_width, const void* kcache,
                                int page_size, int T, int H, int R, int Dr, float scale, int n_splits, float* part_o,
-                               float* part_ml, int* arrivals, hipStream_t stream) {
+                               float* part_ml, int* arrivals, int window, const float* sinks, hipStream_t stream) {
   BLM_REQUIRE(T > 0 && H > 0 && R > 0 && Dr >= 0, "latent_attn: bad sizes T=%d H=%d R=%d Dr=%d", T, H, R, Dr);
   BLM_REQUIRE(R <= LAT_MAX_R, "latent_attn: a latent of %d lanes is more than %d", R, LAT_MAX_R);
-  BLM_REQUIRE(page_size > 0 && table_width > 0, "latent_attn: bad cache geometry");
+  BLM_REQUIRE(page_size > 0 && table_width > 0 && window >= 0, "latent_attn: bad cache geometry");
   BLM_REQUIRE(n_splits >= 1 && n_splits <= 65535 && (n_splits == 1 || (part_o && part_ml && arrivals)),
               "latent_attn: %d splits need their workspace", n_splits);
   const long long items = (long long)T * H;
@@ -403,10 +409,10 @@ extern "C" int blm_latent_attn(const float* qabs, float* olat, int cache_dtype, 
   dim3 grid((unsigned)blocks, (unsigned)n_splits), block(LAT_WAVES * BLM_WAVE);
   if (cache_dtype == BLM_F32)
     hipLaunchKernelGGL(latent_attn_kernel<float>, grid, block, smem, stream, qabs, olat, positions, token_seq, block_table,
-                       table_width, (const float*)kcache, page_size, T, H, R, Dr, scale, n_splits, part_o, part_ml, arrivals);
+                       table_width, (const float*)kcache, page_size, T, H, R, Dr, scale, n_splits, part_o, part_ml, arrivals, window, sinks);
   else if (cache_dtype == BLM_BF16)
     hipLaunchKernelGGL(latent_attn_kernel<bf16>, grid, block, smem, stream, qabs, olat, positions, token_seq, block_table,
-                       table_width, (const bf16*)kcache, page_size, T, H, R, Dr, scale, n_splits, part_o, part_ml, arrivals);
+                       table_width, (const bf16*)kcache, page_size, T, H, R, Dr, scale, n_splits, part_o, part_ml, arrivals, window, sinks);
   else
     return blm_fail("latent_attn: unsupported dtype %d", cache_dtype);
   BLM_LAUNCH_CHECK("latent_attn");
@@ -450,7 +456,8 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
     latent_attn_mfma_kernel(const bf16* __restrict__ q, float* __restrict__ olat, const int* __restrict__ cu_seqlens,
                             const int* __restrict__ lens_after, const int* __restrict__ block_table, int table_width,
                             const bf16* __restrict__ kcache, const bf16* __restrict__ vcache, int B, int H,
-                            int tiles_per_seq, float scale2, int n_splits, float* part_o, float* part_ml) {
+                            int tiles_per_seq, float scale2, int n_splits, float* part_o, float* part_ml, int window,
+                            const float* __restrict__ sinks) {
   constexpr int W = R + DR;
   constexpr int KS = (W + 31) / 32;
   constexpr int DT = R / 16;
@@ -476,9 +483,12 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
   const int last_idx = min(tile * 16 + 15, n_cols - 1);
   const int max_qpos = past + last_idx / H;
   const int max_key = after - 1;
-  const int n_pages = max_qpos / 64 + 1;
+  const int min_qpos = past + (tile * 16) / H;                   // and the first one reaches furthest back
+  const int p_lo = (window > 0 && min_qpos - window + 1 > 0) ? (min_qpos - window + 1) / 64 : 0;
+  const int n_pages = max_qpos / 64 + 1 - p_lo;
   const int per = (n_pages + n_splits - 1) / n_splits;
-  const int p_begin = split * per, p_end = min(n_pages, p_begin + per);
+  const int p_begin = p_lo + split * per, p_end = min(p_lo + n_pages, p_begin + per);
+  const int lo = window > 0 ? qpos - window + 1 : 0;
   const int* bt = block_table + (size_t)b * table_width;
 
   uint4 qf[KS];
@@ -490,8 +500,9 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
       qf[ks] = (valid && (W % 32 == 0 || d < W)) ? *reinterpret_cast<const uint4*>(qrow + d) : make_uint4(0u, 0u, 0u, 0u);
     }
   }
-  float m = -INFINITY;
-  lat_f32x4 l = {0.f, 0.f, 0.f, 0.f};
+  const bool sunk = valid && sinks != nullptr && split == 0;      // a sink counts once
+  float m = sunk ? sinks[head] * 1.4426950408889634f : -INFINITY;
+  lat_f32x4 l = sunk ? lat_f32x4{1.f, 1.f, 1.f, 1.f} : lat_f32x4{0.f, 0.f, 0.f, 0.f};
   lat_f32x4 o[DT];
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) o[dt] = lat_f32x4{0.f, 0.f, 0.f, 0.f};
@@ -519,7 +530,7 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int kj = key0 + lat_key_of(t, kg * 4 + r);
-        s[t][r] = kj <= qpos ? acc[r] : -INFINITY;      // whatever the rows past the data hold, it is replaced here
+        s[t][r] = (kj <= qpos && kj >= lo) ? acc[r] : -INFINITY;      // whatever the rows past the data hold, it is replaced here
       }
     }
     float mx = -INFINITY;
@@ -641,9 +652,10 @@ extern "C" int blm_latent_attn_mfma_supported(int R, int Dr) {
 extern "C" int blm_latent_attn_mfma(const void* q, float* olat, const int* cu_seqlens, const int* lens_after,
                                     const int* block_table, int table_width, const void* kcache, const void* vcache,
                                     int page_size, int B, int max_new, int H, int R, int Dr, float scale, int n_splits,
-                                    float* part_o, float* part_ml, hipStream_t stream) {
+                                    float* part_o, float* part_ml, int window, const float* sinks, hipStream_t stream) {
   BLM_REQUIRE(B > 0 && max_new > 0 && H > 0, "latent_attn_mfma: bad sizes B=%d max_new=%d H=%d", B, max_new, H);
-  BLM_REQUIRE(page_size == 64 && table_width > 0, "latent_attn_mfma: pages of 64 rows");
+  BLM_REQUIRE(page_size == 64 && table_width > 0 && window >= 0, "latent_attn_mfma: pages of 64 rows");
+  BLM_REQUIRE(scale > 0.f, "latent_attn_mfma: the score scale must be positive (got %g)", (double)scale);
   BLM_REQUIRE(n_splits >= 1 && n_splits <= LATM_MAX_PIECES && (n_splits == 1 || (part_o && part_ml)),
               "latent_attn_mfma: %d pieces (1 to %d, with their workspace)", n_splits, LATM_MAX_PIECES);
   const long long tiles = ((long long)max_new * H + 15) / 16;
@@ -656,7 +668,7 @@ extern "C" int blm_latent_attn_mfma(const void* q, float* olat, const int* cu_se
   if (R == r && Dr == d) {                                                                                             \
     hipLaunchKernelGGL((latent_attn_mfma_kernel<r, d>), grid, dim3(LATM_WAVES * BLM_WAVE), 0, stream, (const bf16*)q,  \
                        olat, cu_seqlens, lens_after, block_table, table_width, (const bf16*)kcache, (const bf16*)vcache, \
-                       B, H, (int)tiles, scale2, n_splits, part_o, part_ml);                                           \
+                       B, H, (int)tiles, scale2, n_splits, part_o, part_ml, window, sinks);                            \
     BLM_LAUNCH_CHECK("latent_attn_mfma");                                                                              \
     if (n_splits > 1) {                                                                                                \
       hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)(waves * 16)), dim3(LATM_MERGE_THREADS), 0, stream, part_o, part_ml, \

@@ -10,7 +10,7 @@ import torch
 
 from . import build as _build
 
-ABI_VERSION = 40
+ABI_VERSION = 41
 _lib = None
 _lock = threading.Lock()
 
@@ -46,6 +46,12 @@ _SIGNATURES = {
     "blm_qkv_prepare": [_c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int,
                         _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                         _c_void_p, _c_int, _c_float, _c_void_p],
+    "blm_qkv_norm": [_c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int,
+                     _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_float, _c_float, _c_int, _c_int,
+                     _c_void_p, _c_int, _c_void_p],
+    "blm_head_gate": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+    "blm_map_difference": [_c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void_p],
+    "blm_moe_table": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_int, _c_int, _c_void_p],
     "blm_sigmoid_gate": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "blm_gelu_glu": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
     "blm_softcap": [_c_void_p, ctypes.c_longlong, _c_float, _c_void_p],
@@ -59,7 +65,7 @@ _SIGNATURES = {
     "blm_moe_gate_clamped": [_c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float,
                              _c_void_p],
     "blm_relu2": [_c_void_p, _c_void_p, _c_int, ctypes.c_longlong, _c_void_p],
-    "blm_post_norm": [_c_void_p] + [_c_void_p, _c_int, _c_int, ctypes.c_longlong, _c_float, _c_void_p, _c_float] * 2
+    "blm_post_norm": [_c_void_p] + [_c_void_p, _c_int, _c_int, ctypes.c_longlong, _c_float, _c_void_p, _c_float, _c_void_p] * 2
                      + [_c_void_p, _c_float, _c_int, _c_void_p, _c_int, _c_void_p, _c_float, _c_void_p, _c_int, _c_int, _c_void_p,
                         _c_int, _c_int, _c_void_p],
     "blm_sum_planes": [_c_void_p, _c_int, ctypes.c_longlong, _c_void_p, _c_void_p],
@@ -113,12 +119,12 @@ _SIGNATURES = {
                        _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p],
     "blm_attn_decode": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int,
                         _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int,
-                        _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_float, _c_void_p],
+                        _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_float, _c_int, _c_void_p],
     "blm_attn_decode_supported": [_c_int, _c_int, _c_int],
     "blm_attn_prefill_mfma_supported": [_c_int, _c_int, _c_int],
     "blm_attn_prefill_mfma": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int,
                               _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
-                              _c_int, _c_int, _c_void_p, _c_int, _c_float, _c_void_p],
+                              _c_int, _c_int, _c_void_p, _c_int, _c_float, _c_int, _c_void_p],
     "blm_gemm_tiled": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int,
                        _c_int, _c_int, _c_void_p],
     "blm_gemv_skinny": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int,
@@ -431,38 +437,38 @@ def attn_prefill_mfma(q, q_row_stride, out, positions, cu_seqlens, block_table, 
     Rows cu_seqlens[b] .. cu_seqlens[b+1] of q and out belong to sequence b; max_new is the most
     rows any sequence has.  queries: 16 or 32 query rows per wavefront (attn_prefill_queries chooses).
     sinks (float32 [heads]): the softmax's denominator also holds exp(sinks[h]), a logit without key or value.
-    keep_first: a sequence's first keys that stay visible before the window; softcap c > 0: scores s <- c tanh(s / c)."""
+    out: in q's dtype, or float32 (results that are combined before they are rounded).  keep_first: a sequence's first keys that stay visible before the window; softcap c > 0: scores s <- c tanh(s / c)."""
     _gpu(q, out, positions, cu_seqlens, block_table, kcache, vcache, sinks)
     if sinks is not None:
         _f32("sinks", sinks, nh)
     T = out.shape[0]
     _contig("out", out); _contig("kcache", kcache); _contig("vcache", vcache)
-    if out.shape[1] != nh * hd or out.dtype != q.dtype or kcache.dtype != q.dtype:
-        raise KernelError("attn_prefill_mfma: out must be [T, heads*head_dim] and share q's dtype with the cache")
+    if out.shape[1] != nh * hd or out.dtype not in (q.dtype, torch.float32) or kcache.dtype != q.dtype:
+        raise KernelError("attn_prefill_mfma: out must be [T, heads*head_dim] in q's dtype or float32, the cache in q's dtype")
     if q.stride(-1) != 1 or q_row_stride < nh * hd:
         raise KernelError("attn_prefill_mfma: q rows must be contiguous and at least heads*head_dim long")
     _check_planes("attn_prefill_mfma", kcache, vcache, nkv, page_size, hd)
     _i32("positions", positions, T); _i32("cu_seqlens", cu_seqlens, n_seqs + 1); _i32("block_table", block_table)
     if block_table.shape[0] < n_seqs:
         raise KernelError("attn_prefill_mfma: the page table has fewer rows than there are sequences")
-    _call("blm_attn_prefill_mfma", q.data_ptr(), q_row_stride, out.data_ptr(), _code(out), positions.data_ptr(),
+    _call("blm_attn_prefill_mfma", q.data_ptr(), q_row_stride, out.data_ptr(), _code(q), positions.data_ptr(),
           cu_seqlens.data_ptr(), block_table.data_ptr(), block_table.shape[1], kcache.data_ptr(), vcache.data_ptr(),
           page_size, int(n_seqs), int(max_new), nh, nkv, hd, float(scale), int(window), int(queries), _ptr(sinks),
-          int(keep_first), float(softcap), _stream())
+          int(keep_first), float(softcap), 1 if out.dtype == torch.float32 else 0, _stream())
     return out
 
 
 def attn_decode(q, q_row_stride, out, positions, token_seq, block_table, kcache, vcache, page_size,
                 nh, nkv, hd, scale, window=0, n_splits=1, sinks=None, keep_first=0, softcap=0.0):
-    """Attention for few query tokens over long key ranges, the key range cut into n_splits.  sinks, keep_first,
+    """Attention for few query tokens over long key ranges, the key range cut into n_splits.  out, sinks, keep_first,
     softcap: as for attn_prefill_mfma."""
     _gpu(q, out, positions, token_seq, block_table, kcache, vcache, sinks)
     if sinks is not None:
         _f32("sinks", sinks, nh)
     T = out.shape[0]
     _contig("out", out); _contig("kcache", kcache); _contig("vcache", vcache)
-    if out.shape[1] != nh * hd or out.dtype != q.dtype or kcache.dtype != q.dtype:
-        raise KernelError("attn_decode: out must be [T, heads*head_dim] and share q's dtype with the cache")
+    if out.shape[1] != nh * hd or out.dtype not in (q.dtype, torch.float32) or kcache.dtype != q.dtype:
+        raise KernelError("attn_decode: out must be [T, heads*head_dim] in q's dtype or float32, the cache in q's dtype")
     if q.stride(-1) != 1 or q_row_stride < nh * hd:
         raise KernelError("attn_decode: q rows must be contiguous and at least heads*head_dim long")
     _check_planes("attn_decode", kcache, vcache, nkv, page_size, hd)
@@ -473,10 +479,10 @@ def attn_decode(q, q_row_stride, out, positions, token_seq, block_table, kcache,
         part_o = torch.empty(T * nh * n_splits * hd, dtype=torch.float32, device=out.device)
         part_ml = torch.empty(T * nh * n_splits * 2, dtype=torch.float32, device=out.device)
         arrivals = arrival_counters(out.device)
-    _call("blm_attn_decode", q.data_ptr(), q_row_stride, out.data_ptr(), _code(out), positions.data_ptr(),
+    _call("blm_attn_decode", q.data_ptr(), q_row_stride, out.data_ptr(), _code(q), positions.data_ptr(),
           token_seq.data_ptr(), block_table.data_ptr(), block_table.shape[1], kcache.data_ptr(), vcache.data_ptr(),
           page_size, T, nh, nkv, hd, float(scale), int(window), n_splits, _ptr(part_o), _ptr(part_ml),
-          _ptr(arrivals), _ptr(sinks), int(keep_first), float(softcap), _stream())
+          _ptr(arrivals), _ptr(sinks), int(keep_first), float(softcap), 1 if out.dtype == torch.float32 else 0, _stream())
     return out
 
 
@@ -1012,10 +1018,14 @@ def latent_attn_max_splits(T, H, R):
 
 
 
-def latent_attn(qabs, olat, kcache, step, block_table, page_size, H, R, Dr, scale, n_splits=1):
+def latent_attn(qabs, olat, kcache, step, block_table, page_size, H, R, Dr, scale, n_splits=1, window=0, sinks=None):
     """softmax over each query's visible rows of (qabs . [latent | key lanes]) * scale, times the latents:
-    olat float32 [T, H, R].  qabs float32 [T, H, R + Dr]; kcache [pages, 1, page, R + Dr]."""
-    _gpu(qabs, olat, kcache, block_table)
+    olat float32 [T, H, R].  qabs float32 [T, H, R + Dr]; kcache [pages, 1, page, R + Dr].  window: row j is visible to
+    position p while p - j < window (0: every earlier row).  sinks (float32 [H] or None): exp(sinks[h]) is part of the
+    denominator."""
+    _gpu(qabs, olat, kcache, block_table, sinks)
+    if sinks is not None:
+        _f32("sinks", sinks, H)
     T = qabs.shape[0]
     _f32("qabs", qabs, T * H * (R + Dr)); _f32("olat", olat, T * H * R)
     _contig("kcache", kcache); _i32("block_table", block_table)
@@ -1031,7 +1041,7 @@ def latent_attn(qabs, olat, kcache, step, block_table, page_size, H, R, Dr, scal
         arrivals = arrival_counters(qabs.device)
     _call("blm_latent_attn", qabs.data_ptr(), olat.data_ptr(), _code(kcache), step.positions.data_ptr(),
           step.token_seq.data_ptr(), block_table.data_ptr(), block_table.shape[1], kcache.data_ptr(), page_size, T, H, R,
-          Dr, float(scale), n_splits, _ptr(part_o), _ptr(part_ml), _ptr(arrivals), _stream())
+          Dr, float(scale), n_splits, _ptr(part_o), _ptr(part_ml), _ptr(arrivals), int(window), _ptr(sinks), _stream())
     return olat
 
 
@@ -1045,10 +1055,12 @@ def latent_attn_mfma_max_splits(n_seqs, max_new, H, R):
     return max(1, LATENT_SCRATCH_FLOATS // (waves * 16 * (R + 2)))
 
 
-def latent_attn_mfma(q, olat, kcache, vcache, step, block_table, page_size, H, R, Dr, scale, n_splits=1):
+def latent_attn_mfma(q, olat, kcache, vcache, step, block_table, page_size, H, R, Dr, scale, n_splits=1, window=0, sinks=None):
     """The same function as latent_attn on the matrix cores: q bfloat16 [T, H, R + Dr], key pages and transposed
     latent pages ([pages, 1, R, 64]) in bfloat16; olat float32 [T, H, R]."""
-    _gpu(q, olat, kcache, vcache, block_table)
+    _gpu(q, olat, kcache, vcache, block_table, sinks)
+    if sinks is not None:
+        _f32("sinks", sinks, H)
     T = q.shape[0]
     _contig("q", q); _contig("kcache", kcache); _contig("vcache", vcache); _i32("block_table", block_table)
     _f32("olat", olat, T * H * R)
@@ -1067,7 +1079,7 @@ def latent_attn_mfma(q, olat, kcache, vcache, step, block_table, page_size, H, R
         part_o, part_ml = buf[: cols * n_splits * R], buf[cols * n_splits * R: cols * n_splits * (R + 2)]
     _call("blm_latent_attn_mfma", q.data_ptr(), olat.data_ptr(), step.cu_seqlens.data_ptr(), step.lens_after.data_ptr(),
           block_table.data_ptr(), block_table.shape[1], kcache.data_ptr(), vcache.data_ptr(), page_size, step.n_seqs,
-          step.max_new, H, R, Dr, float(scale), n_splits, _ptr(part_o), _ptr(part_ml), _stream())
+          step.max_new, H, R, Dr, float(scale), n_splits, _ptr(part_o), _ptr(part_ml), int(window), _ptr(sinks), _stream())
     return olat
 
 
@@ -1262,6 +1274,83 @@ def sigmoid_gate(x, gate):
     return x
 
 
+def qkv_norm(qkv, bias, q_weight, k_weight, eps, step, block_table, kcache, vcache, page_size, H, G, dk, dv, whole_rows=False,
+             growth=None, q_out=None):
+    """Bias, RMS norm and page write between a q/k/v projection and an attention without rotation.  qkv [T, >= (H + G) dk +
+    values]: H query and G key heads of dk lanes, then the values.  Queries and keys (with their biases) are divided by the
+    root mean square of a head's lanes, or with whole_rows of all their heads' lanes together, times the weights (float32
+    [dk], or [H dk] and [G dk]; None: ones).  growth (coef, every): queries at position p times 1 + coef *
+    ln((p + 1) // every + 1).  Queries go back in place, keys and values into the pages [pages, G, page, dk] and [pages, G,
+    dv, page].
+    q_out [T, 2 H dk]: two maps per head.  Heads 2 h and 2 h + 1 of queries and keys are the maps of head h; keys lie in
+    pages [pages, G / 2, page, 2 dk] side by side, values in [pages, G / 2, dv, page], and query head s goes to
+    q_out[:, s * 2 dk ..] at its map's half of the lanes, zeros in the other half."""
+    _gpu(qkv, bias, q_weight, k_weight, block_table, kcache, vcache, q_out)
+    T, maps = qkv.shape[0], 1 if q_out is None else 2
+    need = (H + G) * dk + G // maps * dv
+    if qkv.stride(1) != 1 or qkv.shape[1] < need or T != step.n_tokens:
+        raise KernelError(f"qkv_norm: rows of {qkv.shape[1]}, needs {need} contiguous ones")
+    if maps == 2 and (H % 2 or G % 2 or whole_rows or q_out.stride(1) != 1 or tuple(q_out.shape) != (T, 2 * H * dk) or q_out.dtype != qkv.dtype):
+        raise KernelError("qkv_norm: two maps per head need an even number of heads, norms per head and queries' rows [T, 2 H dk]")
+    if bias is not None:
+        _f32("bias", bias, need)
+    for name, w, heads in (("query weights", q_weight, H), ("key weights", k_weight, G)):
+        if w is not None:
+            _f32(name, w, heads * dk if whole_rows else dk)
+    _contig("kcache", kcache); _contig("vcache", vcache); _i32("block_table", block_table)
+    if kcache.dtype != qkv.dtype or vcache.dtype != qkv.dtype or tuple(kcache.shape[1:]) != (G // maps, page_size, maps * dk) \
+            or tuple(vcache.shape) != (kcache.shape[0], G // maps, dv, page_size):
+        raise KernelError(f"qkv_norm: pages {tuple(kcache.shape)} / {tuple(vcache.shape)} do not fit")
+    coef, every = growth or (0.0, 0)
+    _call("blm_qkv_norm", qkv.data_ptr(), _code(qkv), qkv.stride(0), _ptr(bias), step.positions.data_ptr(), step.token_seq.data_ptr(),
+          block_table.data_ptr(), block_table.shape[1], kcache.data_ptr(), vcache.data_ptr(), page_size, T, H, G, dk, dv,
+          1 if whole_rows else 0, _ptr(q_weight), _ptr(k_weight), float(eps), float(coef), int(every), maps, _ptr(q_out),
+          q_out.stride(0) if q_out is not None else 0, _stream())
+    return qkv if q_out is None else q_out
+
+
+def head_gate(x, gate, dv):
+    """x[t, h * dv + d] *= sigmoid(gate[t, h]) in place; x [T, H dv], gate [T, H], contiguous rows of any stride, one dtype."""
+    _gpu(x, gate)
+    T, H = gate.shape
+    if tuple(x.shape) != (T, H * dv) or x.stride(1) != 1 or gate.stride(1) != 1 or x.dtype != gate.dtype:
+        raise KernelError("head_gate: x is [T, H dv] and gate [T, H] with contiguous rows in one dtype")
+    _call("blm_head_gate", x.data_ptr(), x.stride(0), gate.data_ptr(), gate.stride(0), _code(x), T, H, dv, _stream())
+    return x
+
+
+def map_difference(a, out, step, H, dv, lam, eps, factor):
+    """out[t, h] = u / sqrt(mean(u^2) + eps) * factor with u = a[t, 2 h] - lam * a[t, 2 h + 1] over dv lanes; a float32
+    [T, 2 H dv], out [T, H dv].  Rows of tokens of no sequence become zero."""
+    _gpu(a, out)
+    T = out.shape[0]
+    _f32("a", a, T * 2 * H * dv); _contig("out", out)
+    if tuple(out.shape) != (T, H * dv) or a.numel() != T * 2 * H * dv or T != step.n_tokens:
+        raise KernelError(f"map_difference: {tuple(a.shape)} and {tuple(out.shape)} do not fit")
+    _call("blm_map_difference", a.data_ptr(), out.data_ptr(), _code(out), step.token_seq.data_ptr(), T, H, dv, float(lam), float(eps),
+          float(factor), _stream())
+    return out
+
+
+def moe_table(table, ids, weights, n_experts, token_source=None):
+    """weights [T, E + 1] float32: 1 / top where table[id of token t] (int32 [vocabulary, top]) names the expert, zero
+    elsewhere, one at E.  token_source: None or the step's (rows, cell) of tokens that are still on the device."""
+    _gpu(table, ids, weights)
+    T = weights.shape[0]
+    _i32("table", table); _i32("ids", ids, T); _f32("weights", weights, T * (n_experts + 1))
+    if table.dim() != 2 or tuple(weights.shape) != (T, n_experts + 1):
+        raise KernelError("moe_table: table [vocabulary, top], weights [T, E + 1]")
+    rows = cell = None
+    if token_source is not None:
+        rows, cell = token_source
+        _i32("source_rows", rows, T)
+        if cell.dtype != torch.int64 or cell.numel() != 1:
+            raise KernelError("moe_table: the cell is one int64 on the device")
+    _call("blm_moe_table", table.data_ptr(), ids.data_ptr(), _ptr(rows), _ptr(cell), table.shape[0], table.shape[1],
+          weights.data_ptr(), T, n_experts, _stream())
+    return weights
+
+
 def moe_route(logits, bias, n_experts, top, shared_col, weights):
     """weights [T, E + 1] float32: for each token the softmax over its `top` largest of (logits[:, :E] + bias) at the
     chosen experts' places and zero elsewhere; at E the sigmoid of logits[:, shared_col] (shared_col < 0: one)."""
@@ -1348,8 +1437,8 @@ def post_norm(h, terms, post=None, fresh=False, vec=None, write_h=True, gamma=No
         v = (0 if fresh else h[r]) + vec + y;  h[r] = v if write_h
         out[i] = n(v, eps) * gamma, or v where gamma is None            (out None: the residual alone)
     with n(x, eps) = x / sqrt(mean(x^2) + eps) and r = rows[i] if rows is given, else i.  terms: up to two of
-    (y, scale, gamma, eps), y [T, D] in a kernel dtype or float32 planes [P, T, D] that are summed.  Weights and vec are
-    float32 [D].  out [n, D] may be a view of wider rows."""
+    (y, scale, gamma, eps) or (y, scale, gamma, eps, bias), y [T, D] in a kernel dtype or float32 planes [P, T, D] that are
+    summed, bias (or None) added to it first.  Weights, biases and vec are float32 [D].  out [n, D] may be a view of wider rows."""
     _gpu(h, vec, gamma, out, rows)
     if h.dtype != torch.float32 or h.dim() != 2:
         raise KernelError("post_norm: the residual stream must be float32 [T, D]")
@@ -1358,14 +1447,17 @@ def post_norm(h, terms, post=None, fresh=False, vec=None, write_h=True, gamma=No
     if not 1 <= len(terms) <= MAX_NORMED_TERMS:
         raise KernelError(f"post_norm: {len(terms)} results (1 to {MAX_NORMED_TERMS})")
     args = []
-    for y, scale, g, e in terms:
-        _gpu(y, g)
+    for y, scale, g, e, *rest in terms:
+        bias = rest[0] if rest else None
+        _gpu(y, g, bias)
         planes, code = _planes("post_norm", y, T, D)
         if g is not None:
             _f32("gamma of a result", g, D)
-        args += [y.data_ptr(), code, planes, T * D, float(scale), _ptr(g), float(e)]
+        if bias is not None:
+            _f32("bias of a result", bias, D)
+        args += [y.data_ptr(), code, planes, T * D, float(scale), _ptr(g), float(e), _ptr(bias)]
     if len(terms) == 1:
-        args += [0, 0, 1, 0, 0.0, 0, 0.0]
+        args += [0, 0, 1, 0, 0.0, 0, 0.0, 0]
     if post is not None:
         _gpu(post[0]); _f32("post gamma", post[0], D)
     for name, v in (("vec", vec), ("gamma", gamma)):
@@ -1662,12 +1754,14 @@ def sink_attn(q, out, sinks, mix, step, block_table, kcache, vcache, page_size, 
               softcap=0.0):
     """Attention whose softmax denominator also holds exp(sinks[h]) (sinks None: a plain softmax) and whose weights
     are mixed between heads by mix [H, H] (None: not mixed) before head h reads the values of its own key-value head.
-    q [T, >= H dk] rows (queries already rotated), out [T, H * dv] in q's dtype.  keep_first: a sequence's first keys
+    q [T, >= H dk] rows (queries already rotated), out [T, H * dv] in q's dtype, or float32 for unmixed heads (rows of
+    tokens of no sequence then hold anything).  keep_first: a sequence's first keys
     that stay visible before the window; softcap c > 0: scores s <- c tanh(s / c)."""
     _gpu(q, out, sinks, mix, block_table, kcache, vcache)
     T = q.shape[0]
     _contig("out", out); _contig("kcache", kcache); _contig("vcache", vcache); _i32("block_table", block_table)
-    if q.stride(1) != 1 or out.dtype != q.dtype or kcache.dtype != q.dtype or vcache.dtype != q.dtype:
+    raw = mix is None and out.dtype == torch.float32      # the kernel's own float results
+    if q.stride(1) != 1 or not (raw or out.dtype == q.dtype) or kcache.dtype != q.dtype or vcache.dtype != q.dtype:
         raise KernelError("sink_attn: queries, pages and output share a dtype; rows contiguous")
     if tuple(out.shape) != (T, H * dv) or tuple(kcache.shape[1:]) != (G, page_size, dk) \
             or tuple(vcache.shape) != (kcache.shape[0], G, dv, page_size) or T != step.n_tokens:
@@ -1676,8 +1770,8 @@ def sink_attn(q, out, sinks, mix, step, block_table, kcache, vcache, page_size, 
         _f32("sinks", sinks, H)
     if mix is not None:
         _f32("mix", mix, H * H)
-    A = torch.empty(T, H, G if mix is not None else 1, dv, dtype=torch.float32, device=q.device)
-    _call("blm_sink_attn", q.data_ptr(), q.stride(0), out.data_ptr(), _code(q), A.data_ptr(), _ptr(sinks), _ptr(mix),
+    A = out if raw else torch.empty(T, H, G if mix is not None else 1, dv, dtype=torch.float32, device=q.device)
+    _call("blm_sink_attn", q.data_ptr(), q.stride(0), 0 if raw else out.data_ptr(), _code(q), A.data_ptr(), _ptr(sinks), _ptr(mix),
           step.positions.data_ptr(), step.token_seq.data_ptr(), block_table.data_ptr(), block_table.shape[1],
           kcache.data_ptr(), vcache.data_ptr(), page_size, T, H, G, dk, dv, float(scale), int(window), int(keep_first),
           float(softcap), _stream())
@@ -1718,7 +1812,8 @@ def sink_attn_mfma(q, out, sinks, mix, step, block_table, kcache, vcache, page_s
     sink_attn_mfma_init(q.device)
     T = q.shape[0]
     _contig("out", out); _contig("kcache", kcache); _contig("vcache", vcache); _i32("block_table", block_table)
-    if q.stride(1) != 1 or not (q.dtype == out.dtype == kcache.dtype == vcache.dtype == torch.bfloat16):
+    raw = mix is None and out.dtype == torch.float32      # the kernel's own float results
+    if q.stride(1) != 1 or not (q.dtype == kcache.dtype == vcache.dtype == torch.bfloat16) or not (raw or out.dtype == q.dtype):
         raise KernelError("sink_attn_mfma: queries, pages and output in bfloat16; rows contiguous")
     if tuple(out.shape) != (T, H * dv) or tuple(kcache.shape[1:]) != (G, page_size, dk) \
             or tuple(vcache.shape) != (kcache.shape[0], G, dv, page_size) or T != step.n_tokens \
@@ -1729,7 +1824,7 @@ def sink_attn_mfma(q, out, sinks, mix, step, block_table, kcache, vcache, page_s
     if mix is not None:
         _f32("mix", mix, H * H)
     n_out = G if mix is not None else 1
-    A = torch.empty(T, H, n_out, dv, dtype=torch.float32, device=q.device)
+    A = out if raw else torch.empty(T, H, n_out, dv, dtype=torch.float32, device=q.device)
     part_o = part_ml = None
     if n_splits > 1:
         if n_splits > sink_attn_mfma_max_splits(step.n_seqs, step.max_new, H, G, dv, mix is not None):
@@ -1737,7 +1832,7 @@ def sink_attn_mfma(q, out, sinks, mix, step, block_table, kcache, vcache, page_s
         cols = step.n_seqs * G * ((step.max_new * (H // G) + 15) // 16) * 16
         buf = latent_attn_init(q.device)
         part_o, part_ml = buf[: cols * n_splits * n_out * dv], buf[cols * n_splits * n_out * dv: cols * n_splits * (n_out * dv + 2)]
-    _call("blm_sink_attn_mfma", q.data_ptr(), q.stride(0), out.data_ptr(), A.data_ptr(), _ptr(sinks), _ptr(mix),
+    _call("blm_sink_attn_mfma", q.data_ptr(), q.stride(0), 0 if raw else out.data_ptr(), A.data_ptr(), _ptr(sinks), _ptr(mix),
           step.token_seq.data_ptr(), step.cu_seqlens.data_ptr(), step.lens_after.data_ptr(), block_table.data_ptr(),
           block_table.shape[1], kcache.data_ptr(), vcache.data_ptr(), page_size, step.n_seqs, step.max_new, T, H, G, dk, dv,
           float(scale), int(window), int(n_splits), int(group_batch), _ptr(part_o), _ptr(part_ml), _stream())

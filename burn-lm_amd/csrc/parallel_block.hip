@@ -442,6 +442,37 @@ extern "C" int blm_moe_route(const float* logits, int ld, const float* bias, int
   return 0;
 }
 
+// Routing by a table of the tokens' ids: weights[t][e] = 1 / top where table[id] names expert e, else 0, and one at E
+// (rows as moe_route leaves them).  The token of row t: (*source)[source_rows[t]] where source_rows is given and not
+// negative, else ids[t]; an id outside [0, V) chooses no expert.  A wavefront per token.
+__global__ void __launch_bounds__(256)
+    moe_table_kernel(const int* __restrict__ table, const int* __restrict__ ids, const int* __restrict__ source_rows,
+                     const int* const* __restrict__ source, int V, int top, float* __restrict__ weights, int T, int E) {
+  const int t = blockIdx.x * 4 + threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
+  if (t >= T) return;
+  const int r = source_rows ? source_rows[t] : -1;
+  const int id = r >= 0 ? (*source)[r] : ids[t];
+  const bool good = (unsigned)id < (unsigned)V;
+  const int* row = table + (size_t)(good ? id : 0) * top;
+  const float share = 1.0f / (float)top;
+  for (int e = lane; e <= E; e += BLM_WAVE) {
+    float w = e == E ? 1.0f : 0.f;
+    for (int k = 0; k < top; ++k)
+      if (good && row[k] == e) w = share;
+    weights[(size_t)t * (E + 1) + e] = w;
+  }
+}
+
+extern "C" int blm_moe_table(const int* table, const int* ids, const int* source_rows, const void* source_cell, int V, int top,
+                             float* weights, int T, int E, hipStream_t stream) {
+  BLM_REQUIRE(T > 0 && E > 0 && top > 0 && top <= E && V > 0, "moe_table: bad sizes T=%d E=%d top=%d V=%d", T, E, top, V);
+  BLM_REQUIRE((source_rows == nullptr) == (source_cell == nullptr), "moe_table: rows and cell of a token source come together");
+  hipLaunchKernelGGL(moe_table_kernel, dim3((T + 3) / 4), dim3(256), 0, stream, table, ids, source_rows,
+                     (const int* const*)source_cell, V, top, weights, T, E);
+  BLM_LAUNCH_CHECK("moe_table");
+  return 0;
+}
+
 // The experts' gated activations, each scaled by its expert's weight for the token, for experts that run as one
 // stacked product.  gate_up [T][2 I] with I = E * ffe + ffs columns of gates (expert e at e * ffe, the shared expert
 // behind them), then as many of ups.  out[t][i] = silu(gate) * up * weights[t][expert of column i].

@@ -1,5 +1,6 @@
 // Sublayer results that are normed before they join the residual, and what follows the join, as one kernel per row:
 //
+//   y_i = y_i + (bias_i ? bias_i : 0)                                   a last projection's bias
 //   y = sum_i scale_i * (gamma_i ? n(y_i, eps_i) * gamma_i : y_i)       up to two results (two mixers side by side)
 //   y = post_gamma ? n(y, post_eps) * post_gamma : y                    the norm behind the sublayer
 //   v = (fresh ? 0 : h[r]) + (vec ? vec : 0) + y                        fresh: the residual starts anew from y
@@ -16,6 +17,7 @@
 struct PnTerm {
   const void* y;
   const float* gamma;
+  const float* bias;
   size_t stride;      // elements between planes
   int planes, dtype;
   float scale, eps;
@@ -65,10 +67,10 @@ __device__ __forceinline__ void pn_result4(const PnTerm& t, size_t at, float* v)
       }
   }
 }
-__device__ __forceinline__ float pn_result1(const PnTerm& t, size_t at) {
-  if (t.dtype == BLM_BF16) return to_float(reinterpret_cast<const bf16*>(t.y)[at]);
+__device__ __forceinline__ float pn_result1(const PnTerm& t, size_t at, int d) {
+  float v = t.bias ? t.bias[d] : 0.f;
+  if (t.dtype == BLM_BF16) return v + to_float(reinterpret_cast<const bf16*>(t.y)[at]);
   const float* y = reinterpret_cast<const float*>(t.y) + at;
-  float v = 0.f;
   for (int p = 0; p < t.planes; ++p) v += y[(size_t)p * t.stride];
   return v;
 }
@@ -110,6 +112,12 @@ __global__ void __launch_bounds__(512) post_norm_vec_kernel(float* __restrict__ 
 #pragma unroll
       for (int n = 0; n < NT; ++n) {
         pn_result4(g.term[n], row + d, y[n][it]);
+        if (g.term[n].bias) {
+          float x[4];
+          pn_load4(g.term[n].bias + d, x);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) y[n][it][e] += x[e];
+        }
         if (g.term[n].gamma) pn_load4(g.term[n].gamma + d, w[n][it]);
       }
       if (g.post_gamma) pn_load4(g.post_gamma + d, wp[it]);
@@ -186,7 +194,7 @@ __global__ void __launch_bounds__(256) post_norm_kernel(float* __restrict__ h, T
     float ss[2] = {0.f, 0.f};
     for (int d = threadIdx.x; d < D; d += blockDim.x)
       for (int n = 0; n < g.n_terms; ++n) {
-        const float a = pn_result1(g.term[n], row + d);
+        const float a = pn_result1(g.term[n], row + d, d);
         ss[n] = fmaf(a, a, ss[n]);
       }
     pn_block_sum2(ss[0], ss[1], red[0]);
@@ -195,7 +203,7 @@ __global__ void __launch_bounds__(256) post_norm_kernel(float* __restrict__ h, T
   }
   auto sum_of = [&](int d) {
     float a = 0.f;
-    for (int n = 0; n < g.n_terms; ++n) a = fmaf(pn_result1(g.term[n], row + d) * c[n], g.term[n].gamma ? g.term[n].gamma[d] : 1.f, a);
+    for (int n = 0; n < g.n_terms; ++n) a = fmaf(pn_result1(g.term[n], row + d, d) * c[n], g.term[n].gamma ? g.term[n].gamma[d] : 1.f, a);
     return a;
   };
   float cp = 1.f;
@@ -220,20 +228,20 @@ __global__ void __launch_bounds__(256) post_norm_kernel(float* __restrict__ h, T
   }
 }
 
-// Terms: y, dtype, planes, plane stride, scale, gamma (or null), eps; the second one may have a null y (one term).
+// Terms: y, dtype, planes, plane stride, scale, gamma (or null), eps, bias (or null); the second one may have a null y (one term).
 // out may be null (the residual alone), gamma null (out is the residual's rows as they are).
 extern "C" int blm_post_norm(float* h, const void* y0, int dtype0, int planes0, long long stride0, float scale0, const float* gamma0,
-                             float eps0, const void* y1, int dtype1, int planes1, long long stride1, float scale1,
-                             const float* gamma1, float eps1, const float* post_gamma, float post_eps, int fresh,
+                             float eps0, const float* bias0, const void* y1, int dtype1, int planes1, long long stride1, float scale1,
+                             const float* gamma1, float eps1, const float* bias1, const float* post_gamma, float post_eps, int fresh,
                              const float* vec, int write_h, const float* gamma, float eps, void* out, int act_dtype, int ldo,
                              const int* rows, int n_out, int D, hipStream_t stream) {
   BLM_REQUIRE(h && n_out > 0 && D > 0 && y0 && (out || write_h), "post_norm: bad sizes n=%d D=%d, or nothing to write", n_out, D);
   BLM_REQUIRE(!out || ldo >= D, "post_norm: rows of %d elements do not hold %d", ldo, D);
   PnArgs g;
-  g.term[0] = PnTerm{y0, gamma0, (size_t)stride0, planes0, dtype0, scale0, eps0};
-  g.term[1] = PnTerm{y1, gamma1, (size_t)stride1, planes1, dtype1, scale1, eps1};
+  g.term[0] = PnTerm{y0, gamma0, bias0, (size_t)stride0, planes0, dtype0, scale0, eps0};
+  g.term[1] = PnTerm{y1, gamma1, bias1, (size_t)stride1, planes1, dtype1, scale1, eps1};
   g.n_terms = y1 ? 2 : 1;
-  if (!y1) g.term[1] = PnTerm{y0, nullptr, 0, 1, dtype0, 0.f, 0.f};
+  if (!y1) g.term[1] = PnTerm{y0, nullptr, nullptr, 0, 1, dtype0, 0.f, 0.f};
   for (int n = 0; n < g.n_terms; ++n)
     BLM_REQUIRE(g.term[n].planes >= 1 && (g.term[n].dtype == BLM_F32 || (g.term[n].dtype == BLM_BF16 && g.term[n].planes == 1)),
                 "post_norm: result %d is not float planes or one bfloat16 plane", n);
@@ -245,7 +253,7 @@ extern "C" int blm_post_norm(float* h, const void* y0, int dtype0, int planes0, 
   bool vec4 = D % 4 == 0 && ((uintptr_t)h & 15) == 0 && (!out || (((uintptr_t)out & (4 * esize - 1)) == 0 && ldo % 4 == 0)) &&
               (((uintptr_t)post_gamma | (uintptr_t)vec | (uintptr_t)gamma) & 15) == 0;
   for (int n = 0; n < g.n_terms; ++n)
-    vec4 = vec4 && ((uintptr_t)g.term[n].y & (g.term[n].dtype == BLM_F32 ? 15 : 7)) == 0 && ((uintptr_t)g.term[n].gamma & 15) == 0 &&
+    vec4 = vec4 && ((uintptr_t)g.term[n].y & (g.term[n].dtype == BLM_F32 ? 15 : 7)) == 0 && (((uintptr_t)g.term[n].gamma | (uintptr_t)g.term[n].bias) & 15) == 0 &&
            g.term[n].stride % 4 == 0;
   const int threads = D >= 2048 ? 512 : 256;
   if (vec4 && D <= threads * 16) {

@@ -97,16 +97,35 @@ __global__ void qkv_prepare_kernel(TA* __restrict__ qkv, int ld, const float* __
   }
 }
 
-// The same for unit-norm heads that do not turn: a wavefront per head, whose lanes stay in registers between the norm and
-// the stores (dk up to 64 * QU_LANES).  grid (tokens, blocks of four heads: H queries, then G keys, then, where the values
-// have columns of their own, G values)
+// What is done to normed queries and keys besides the norm:
+//   qw, kw (float or null)   stored weights of the norm, one per lane (of a head, or of the whole row)
+//   coef, every              queries grow with their position p: times 1 + coef * ln(floor((p + 1) / every) + 1)
+//   maps, q_out, ld_q        maps = 2: every query and key head is two of half the page's lanes, [map 1 | map 2].  Keys lie
+//                            in the pages as they come, both maps of a head side by side; query head s of map x goes to
+//                            q_out[t][s * 2 dk ..] at lanes x * dk .. with zeros in the other half, so that its product with
+//                            a page's row is the product with its own map.  maps = 1: q_out null, queries stay in place.
+struct QnExtra {
+  const float* qw;
+  const float* kw;
+  float coef;
+  int every, maps, ld_q;
+  void* q_out;
+};
+__device__ __forceinline__ float qn_growth(const QnExtra& x, int pos) {
+  return x.every > 0 ? 1.0f + x.coef * logf((float)((pos + 1) / x.every + 1)) : 1.0f;
+}
+
+// The same for normed heads that do not turn: a wavefront per head, whose lanes stay in registers between the norm and
+// the stores (dk up to 64 * QU_LANES).  H, G count heads of dk lanes (with two maps: twice the heads of the pages).
+// grid (tokens, blocks of four heads: H queries, then G keys, then, where the values have columns of their own,
+// G / maps values)
 #define QU_LANES 8
 template <typename TA>
 __global__ void __launch_bounds__(256)
     qkv_unit_kernel(TA* __restrict__ qkv, int ld, const float* __restrict__ bias, const int* __restrict__ positions,
                     const int* __restrict__ token_seq, const int* __restrict__ block_table, int table_width, TA* __restrict__ kcache,
                     TA* __restrict__ vcache, int page_size, int H, int G, int dk, int dv, int n_heads, int values_are_keys,
-                    const float* __restrict__ q_scale, float norm_eps) {
+                    const float* __restrict__ q_scale, float norm_eps, QnExtra ex) {
   const int t = blockIdx.x, lane = threadIdx.x & (BLM_WAVE - 1);
   const int head = blockIdx.y * 4 + threadIdx.x / BLM_WAVE;
   if (head >= n_heads) return;
@@ -119,35 +138,131 @@ __global__ void __launch_bounds__(256)
   size_t page = 0;
   if (head >= H) page = block_table[(size_t)b * table_width + pos / page_size];
   const int in_page = pos % page_size;
-  float x[QU_LANES];
+  const float* w = value ? nullptr : head < H ? ex.qw : ex.kw;
+  float x[QU_LANES], g[QU_LANES];
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < QU_LANES; ++k) {
     const int d = lane + k * BLM_WAVE;
     x[k] = d < n ? to_float(row[col + d]) + (bias ? bias[col + d] : 0.f) : 0.f;
+    g[k] = (w && d < n) ? w[d] : 1.0f;
     ss = fmaf(x[k], x[k], ss);
   }
   const float f = value ? 1.0f : 1.0f / sqrtf(wave_sum(ss) / (float)dk + norm_eps);
   if (head < H) {
-    const float fq = f * (q_scale ? q_scale[head] : 1.0f);
+    const float fq = f * (q_scale ? q_scale[head] : 1.0f) * qn_growth(ex, pos);
+    if (ex.maps == 2) {
+      TA* o = (TA*)ex.q_out + (size_t)t * ex.ld_q + (size_t)head * 2 * dk;
+      const int mine = (head & 1) * dk, other = dk - mine;
+#pragma unroll
+      for (int k = 0; k < QU_LANES; ++k) {
+        const int d = lane + k * BLM_WAVE;
+        if (d < n) {
+          o[mine + d] = from_float<TA>(x[k] * g[k] * fq);
+          o[other + d] = from_float<TA>(0.f);
+        }
+      }
+      return;
+    }
 #pragma unroll
     for (int k = 0; k < QU_LANES; ++k) {
       const int d = lane + k * BLM_WAVE;
-      if (d < n) row[col + d] = from_float<TA>(x[k] * fq);
+      if (d < n) row[col + d] = from_float<TA>(x[k] * g[k] * fq);
     }
     return;
   }
-  const int c = value ? head - H - G : head - H;
-  TA* krow = kcache + ((page * G + c) * page_size + in_page) * dk;
-  TA* vcol = vcache + (page * G + c) * (size_t)dv * page_size + in_page;
+  const int c = value ? head - H - G : head - H, Gp = G / ex.maps;       // Gp: key-value heads of the pages
+  TA* krow = kcache + ((page * Gp + c / ex.maps) * page_size + in_page) * (dk * ex.maps) + (c % ex.maps) * dk;
+  TA* vcol = vcache + (page * Gp + c) * (size_t)dv * page_size + in_page;
 #pragma unroll
   for (int k = 0; k < QU_LANES; ++k) {
     const int d = lane + k * BLM_WAVE;
     if (d < n) {
-      if (!value) krow[d] = from_float<TA>(x[k] * f);
+      if (!value) krow[d] = from_float<TA>(x[k] * g[k] * f);
       if (value || values_are_keys) vcol[(size_t)d * page_size] = from_float<TA>(x[k]);
     }
   }
+}
+
+// Queries and keys normed over their whole rows at once (all heads together).  grid (tokens, 3): the queries' part of
+// the row, the keys', the values'; a block per part.
+template <typename TA>
+__global__ void __launch_bounds__(256)
+    qkv_row_norm_kernel(TA* __restrict__ qkv, int ld, const float* __restrict__ bias, const int* __restrict__ positions,
+                        const int* __restrict__ token_seq, const int* __restrict__ block_table, int table_width,
+                        TA* __restrict__ kcache, TA* __restrict__ vcache, int page_size, int H, int G, int dk, int dv,
+                        float norm_eps, QnExtra ex) {
+  __shared__ float red[17];
+  const int t = blockIdx.x, part = blockIdx.y;
+  const int b = token_seq[t];
+  if (b < 0) return;
+  const int col = part == 0 ? 0 : part == 1 ? H * dk : (H + G) * dk, n = part == 0 ? H * dk : part == 1 ? G * dk : G * dv;
+  TA* row = qkv + (size_t)t * ld + col;
+  const float* add = bias ? bias + col : nullptr;
+  const int pos = positions[t];
+  float f = 1.0f;
+  if (part < 2) {
+    float ss = 0.f;
+    for (int d = threadIdx.x; d < n; d += blockDim.x) {
+      const float x = to_float(row[d]) + (add ? add[d] : 0.f);
+      ss = fmaf(x, x, ss);
+    }
+    f = 1.0f / sqrtf(block_sum<true>(ss, red) / (float)n + norm_eps);
+  }
+  if (part == 0) {
+    f *= qn_growth(ex, pos);
+    for (int d = threadIdx.x; d < n; d += blockDim.x)
+      row[d] = from_float<TA>((to_float(row[d]) + (add ? add[d] : 0.f)) * f * (ex.qw ? ex.qw[d] : 1.0f));
+    return;
+  }
+  const size_t page = block_table[(size_t)b * table_width + pos / page_size];
+  const int in_page = pos % page_size;
+  for (int d = threadIdx.x; d < n; d += blockDim.x) {
+    const float x = to_float(row[d]) + (add ? add[d] : 0.f);
+    if (part == 1) {
+      const int c = d / dk, i = d - c * dk;
+      kcache[((page * G + c) * page_size + in_page) * dk + i] = from_float<TA>(x * f * (ex.kw ? ex.kw[d] : 1.0f));
+    } else {
+      vcache[(page * G * (size_t)dv + d) * page_size + in_page] = from_float<TA>(x);
+    }
+  }
+}
+
+// Bias, norm (over a head's lanes, or whole_rows: over all of a token's queries, and of its keys), growth of the queries
+// and the write of keys and values into the pages.  H, G: heads of dk lanes in the row (maps = 2: twice the pages' heads).
+extern "C" int blm_qkv_norm(void* qkv, int dtype, int ld, const float* bias, const int* positions, const int* token_seq,
+                            const int* block_table, int table_width, void* kcache, void* vcache, int page_size, int T, int H,
+                            int G, int dk, int dv, int whole_rows, const float* qw, const float* kw, float norm_eps, float coef,
+                            int every, int maps, void* q_out, int ld_q, hipStream_t stream) {
+  BLM_REQUIRE(T > 0 && H > 0 && G > 0 && dk > 0 && dv > 0, "qkv_norm: bad sizes T=%d H=%d G=%d dk=%d dv=%d", T, H, G, dk, dv);
+  BLM_REQUIRE(maps == 1 || (maps == 2 && !whole_rows && H % 2 == 0 && G % 2 == 0 && q_out && ld_q >= 2 * H * dk),
+              "qkv_norm: %d maps (1, or 2 with norms per head and a place for the queries)", maps);
+  BLM_REQUIRE(ld >= (H + G) * dk + G / maps * dv, "qkv_norm: rows of %d are too short", ld);
+  BLM_REQUIRE(kcache && vcache && block_table && page_size > 0 && table_width > 0, "qkv_norm: the pages are missing");
+  BLM_REQUIRE(dtype == BLM_F32 || dtype == BLM_BF16, "qkv_norm: unsupported dtype %d", dtype);
+  BLM_REQUIRE(whole_rows || (dk <= BLM_WAVE * QU_LANES && dv <= BLM_WAVE * QU_LANES), "qkv_norm: heads of %d and %d lanes (up to %d)",
+              dk, dv, BLM_WAVE * QU_LANES);
+  BLM_REQUIRE(every >= 0, "qkv_norm: queries that grow every %d tokens", every);
+  const QnExtra ex{qw, kw, coef, every, maps, ld_q, q_out};
+#define QN_ROWS(TA)                                                                                                       \
+  hipLaunchKernelGGL(qkv_row_norm_kernel<TA>, dim3(T, 3), dim3(256), 0, stream, (TA*)qkv, ld, bias, positions, token_seq, \
+                     block_table, table_width, (TA*)kcache, (TA*)vcache, page_size, H, G, dk, dv, norm_eps, ex)
+#define QN_HEADS(TA)                                                                                                      \
+  hipLaunchKernelGGL(qkv_unit_kernel<TA>, dim3(T, (n_heads + 3) / 4), dim3(256), 0, stream, (TA*)qkv, ld, bias, positions, \
+                     token_seq, block_table, table_width, (TA*)kcache, (TA*)vcache, page_size, H, G, dk, dv, n_heads, 0,  \
+                     (const float*)nullptr, norm_eps, ex)
+  const int n_heads = H + G + G / maps;
+  if (whole_rows) {
+    if (dtype == BLM_F32) QN_ROWS(float);
+    else QN_ROWS(bf16);
+  } else {
+    if (dtype == BLM_F32) QN_HEADS(float);
+    else QN_HEADS(bf16);
+  }
+#undef QN_ROWS
+#undef QN_HEADS
+  BLM_LAUNCH_CHECK("qkv_norm");
+  return 0;
 }
 
 extern "C" int blm_qkv_prepare(void* qkv, int dtype, int ld, const float* bias, const float* cos_sin, int rot,
@@ -168,10 +283,10 @@ extern "C" int blm_qkv_prepare(void* qkv, int dtype, int ld, const float* bias, 
     const dim3 grid(T, (n_heads + 3) / 4);
     if (dtype == BLM_F32)
       hipLaunchKernelGGL(qkv_unit_kernel<float>, grid, dim3(256), 0, stream, (float*)qkv, ld, bias, positions, token_seq, block_table,
-                         table_width, (float*)kcache, (float*)vcache, page_size, H, G, dk, dv, n_heads, values_are_keys, q_scale, norm_eps);
+                         table_width, (float*)kcache, (float*)vcache, page_size, H, G, dk, dv, n_heads, values_are_keys, q_scale, norm_eps, QnExtra{nullptr, nullptr, 0.f, 0, 1, 0, nullptr});
     else
       hipLaunchKernelGGL(qkv_unit_kernel<bf16>, grid, dim3(256), 0, stream, (bf16*)qkv, ld, bias, positions, token_seq, block_table,
-                         table_width, (bf16*)kcache, (bf16*)vcache, page_size, H, G, dk, dv, n_heads, values_are_keys, q_scale, norm_eps);
+                         table_width, (bf16*)kcache, (bf16*)vcache, page_size, H, G, dk, dv, n_heads, values_are_keys, q_scale, norm_eps, QnExtra{nullptr, nullptr, 0.f, 0, 1, 0, nullptr});
     BLM_LAUNCH_CHECK("qkv_unit");
     return 0;
   }
@@ -237,6 +352,83 @@ extern "C" int blm_sigmoid_gate(void* x, int ld_x, const void* g, int ld_g, int 
   else
     return blm_fail("sigmoid_gate: unsupported dtype %d", dtype);
   BLM_LAUNCH_CHECK("sigmoid_gate");
+  return 0;
+}
+
+// ---------------------------------------------------------------------------------------
+// Output gate with one number per head: x[t][h * dv + d] *= sigmoid(g[t][h]).  A wavefront per (token, head).
+// ---------------------------------------------------------------------------------------
+template <typename TA>
+__global__ void __launch_bounds__(256)
+    head_gate_kernel(TA* __restrict__ x, int ld_x, const TA* __restrict__ g, int ld_g, long long items, int H, int dv) {
+  const long long i = (long long)blockIdx.x * 4 + threadIdx.x / BLM_WAVE;
+  if (i >= items) return;
+  const long long t = i / H;
+  const int h = (int)(i - t * H);
+  const float f = 1.0f / (1.0f + __expf(-to_float(g[(size_t)t * ld_g + h])));
+  TA* row = x + (size_t)t * ld_x + (size_t)h * dv;
+  for (int d = threadIdx.x & (BLM_WAVE - 1); d < dv; d += BLM_WAVE) row[d] = from_float<TA>(to_float(row[d]) * f);
+}
+
+extern "C" int blm_head_gate(void* x, int ld_x, const void* g, int ld_g, int dtype, int T, int H, int dv, hipStream_t stream) {
+  BLM_REQUIRE(T > 0 && H > 0 && dv > 0 && ld_x >= H * dv && ld_g >= H, "head_gate: bad sizes T=%d H=%d dv=%d rows of %d and %d", T, H,
+              dv, ld_x, ld_g);
+  const long long items = (long long)T * H;
+  const unsigned blocks = (unsigned)((items + 3) / 4);
+  if (dtype == BLM_F32)
+    hipLaunchKernelGGL(head_gate_kernel<float>, dim3(blocks), dim3(256), 0, stream, (float*)x, ld_x, (const float*)g, ld_g, items, H, dv);
+  else if (dtype == BLM_BF16)
+    hipLaunchKernelGGL(head_gate_kernel<bf16>, dim3(blocks), dim3(256), 0, stream, (bf16*)x, ld_x, (const bf16*)g, ld_g, items, H, dv);
+  else
+    return blm_fail("head_gate: unsupported dtype %d", dtype);
+  BLM_LAUNCH_CHECK("head_gate");
+  return 0;
+}
+
+// ---------------------------------------------------------------------------------------
+// Two maps of attention to one result per head: u = a[t][2 h] - lambda * a[t][2 h + 1] over dv lanes, then
+// out[t][h] = u / sqrt(mean(u^2) + eps) * factor.  a float [T][2 H][dv]; a wavefront per (token, head) of up to 256 lanes.
+// Rows of no sequence become zero.
+// ---------------------------------------------------------------------------------------
+#define MD_LANES 4
+template <typename TA>
+__global__ void __launch_bounds__(256)
+    map_difference_kernel(const float* __restrict__ a, TA* __restrict__ out, const int* __restrict__ token_seq, long long items,
+                          int H, int dv, float lambda, float eps, float factor) {
+  const int lane = threadIdx.x & (BLM_WAVE - 1);
+  const long long i = (long long)blockIdx.x * 4 + threadIdx.x / BLM_WAVE;
+  if (i >= items) return;
+  const bool live = token_seq[i / H] >= 0;
+  const float* p = a + (size_t)i * 2 * dv;
+  float u[MD_LANES];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < MD_LANES; ++k) {
+    const int d = lane + k * BLM_WAVE;
+    u[k] = (live && d < dv) ? fmaf(-lambda, p[dv + d], p[d]) : 0.f;
+    ss = fmaf(u[k], u[k], ss);
+  }
+  const float f = factor / sqrtf(wave_sum(ss) / (float)dv + eps);
+#pragma unroll
+  for (int k = 0; k < MD_LANES; ++k) {
+    const int d = lane + k * BLM_WAVE;
+    if (d < dv) out[(size_t)i * dv + d] = from_float<TA>(u[k] * f);
+  }
+}
+
+extern "C" int blm_map_difference(const float* a, void* out, int dtype, const int* token_seq, int T, int H, int dv, float lambda,
+                                  float eps, float factor, hipStream_t stream) {
+  BLM_REQUIRE(T > 0 && H > 0 && dv > 0 && dv <= BLM_WAVE * MD_LANES, "map_difference: bad sizes T=%d H=%d dv=%d (up to %d lanes)", T, H, dv,
+              BLM_WAVE * MD_LANES);
+  const long long items = (long long)T * H;
+  const unsigned blocks = (unsigned)((items + 3) / 4);
+  if (dtype == BLM_F32)
+    hipLaunchKernelGGL(map_difference_kernel<float>, dim3(blocks), dim3(256), 0, stream, a, (float*)out, token_seq, items, H, dv, lambda, eps, factor);
+  else if (dtype == BLM_BF16)
+    hipLaunchKernelGGL(map_difference_kernel<bf16>, dim3(blocks), dim3(256), 0, stream, a, (bf16*)out, token_seq, items, H, dv, lambda, eps, factor);
+  else
+    return blm_fail("map_difference: unsupported dtype %d", dtype);
+  BLM_LAUNCH_CHECK("map_difference");
   return 0;
 }
 
@@ -390,6 +582,7 @@ extern "C" int blm_sink_attn(const void* q, int ldq, void* out, int dtype, float
                              const int* positions, const int* token_seq, const int* block_table, int table_width,
                              const void* kcache, const void* vcache, int page_size, int T, int H, int G, int dk, int dv,
                              float scale, int window, int keep_first, float cap, hipStream_t stream) {
+  BLM_REQUIRE(out || !mix, "sink_attn: mixed heads need a place for the results");
   BLM_REQUIRE(keep_first >= 0 && cap >= 0.f, "sink_attn: keep_first %d or cap %g is negative", keep_first, (double)cap);
   BLM_REQUIRE(T > 0 && H > 0 && G > 0 && H % G == 0, "sink_attn: bad sizes T=%d heads=%d kv_heads=%d", T, H, G);
   BLM_REQUIRE(dk > 0 && dk <= SA_MAX_DK && dv > 0 && dv <= 64 * SA_MAX_DV_REGS,
@@ -422,6 +615,7 @@ extern "C" int blm_sink_attn(const void* q, int ldq, void* out, int dtype, float
 #undef SA_PICK
 #undef SA_CASE
   BLM_LAUNCH_CHECK("sink_attn");
+  if (!out) return 0;      // the caller takes the float results
   return launch_talk_mix(A, mix, out, dtype, token_seq, T, H, G, dv, stream);
 }
 
@@ -993,5 +1187,6 @@ extern "C" int blm_sink_attn_mfma(const void* q, int ldq, void* out, float* A, c
                        G, all_groups ? G : 1, dv, (int)tiles, n_splits);
     BLM_LAUNCH_CHECK("sink_merge");
   }
+  if (!out) return 0;      // the caller takes the float results
   return launch_talk_mix(A, mix, out, BLM_BF16, token_seq, T, H, G, dv, stream);
 }

@@ -114,8 +114,9 @@ class Model:
         both = None      # a loop's rows [x; x0]: the embedding leaves its half there
         if self.entry is not None:
             both = self.entry.begin(step.n_tokens, step.token_ids.device)
-        h = self._embed(step, None if both is None else both[:, both.shape[1] // 2:])
-        delta = None
+        h, delta = self._embed(step, None if both is None else both[:, both.shape[1] // 2:]), None
+        if hasattr(self.embedding, "normed"):
+            h, delta = self.embedding.normed(h)
         for i, place in enumerate(self.plan.order):
             if place.turn is not None:
                 delta = self.entry.enter(h, delta, both, place.turn)

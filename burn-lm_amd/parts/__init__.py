@@ -8,6 +8,7 @@ from .channel_delta import ChannelDelta
 from .clamped_glu import ClampedGLU
 from .dense_relu2 import DenseRelu2
 from .dense_xielu import DenseXielu
+from .differential_attention import DifferentialAttention
 from .embedding import Embedding, LMHead
 from .gated_residual import GatedPreNormBlock, GatedPreNormMixerBlock, ResidualGate
 from .gelu_glu import GeluGLU
@@ -24,7 +25,7 @@ from .parallel import (CausalConvInput, LayerScale, ParallelBlock, ParallelMixer
                        ScaledParallelMixerBlock, TokenSide)
 from .post_norm import PostNormBlock, PostNormMixerBlock
 from .rope import RotaryEncoding
-from .routed_experts import GroupedRoutedExperts, RoutedExperts
+from .routed_experts import GroupedRoutedExperts, RoutedExperts, TableExperts
 from .sink_attention import SinkAttention
 from .streams import HyperBlock, HyperConnection, HyperMixerBlock
 from .swiglu import SwiGLU
@@ -67,3 +68,5 @@ registry.register_part("feed_forward", "dense_relu2", DenseRelu2)
 registry.register_part("block", "post_norm", PostNormBlock)
 registry.register_part("block", "post_norm_mixer_only", PostNormMixerBlock)
 registry.register_part("connection", "loop_entry", LoopEntry)
+registry.register_part("mixer", "differential_attention", DifferentialAttention)
+registry.register_part("feed_forward", "table_experts", TableExperts)

@@ -90,13 +90,22 @@ class Term:
     """One summand of a sublayer's result, for a block that adds the summands to the residual itself (in float32, each
     with coefficients of its own): ``scale * row[t] * y[t, :]``.  y: [tokens, width] in the activation dtype, or float32
     planes [planes, tokens, width] that are summed; row: float32 [tokens] (any stride) or None.  gamma (float32 [width]
-    or None): y is RMS-normed over its width with this weight and eps before the scale (only for a block that joins its
-    results as a Joining)."""
+    or None): y is RMS-normed over its width with this weight and eps before the scale; bias (float32 [width] or None): the
+    last projection's, added to y first (a block that joins its results as a Joining takes both; summed() is y with its
+    bias for others)."""
     y: torch.Tensor
     scale: float = 1.0
     row: torch.Tensor = None
     gamma: torch.Tensor = None
     eps: float = 0.0
+    bias: torch.Tensor = None
+
+    def summed(self):
+        """y with its bias, for a block that adds plain results."""
+        if self.bias is None:
+            return self.y
+        y = self.y.sum(0) if self.y.dim() == 3 else self.y.float()
+        return (y + self.bias).unsqueeze(0)
 
 
 @dataclass

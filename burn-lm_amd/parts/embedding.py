@@ -10,18 +10,23 @@ import math
 
 import torch
 
-from .base import Part, TensorSpec
+from .base import Joining, Part, TensorSpec, Term
 
 
 class Embedding(Part):
     """params: vocab, width, copies (default 1; more: the residual starts as that many equal streams,
     [tokens, copies, width]), scale (default 1: every row is multiplied by it), position_base (default none; a number b: a
     sinusoidal vector of the token's position p is added, entry 2i the sine and entry 2i + 1 the cosine of
-    p * b^(-2i/width); the angles are reduced in double precision).  names: weight."""
+    p * b^(-2i/width); the angles are reduced in double precision), norm_eps (default none; a number: the looked-up rows
+    pass an RMS norm with this eps before they are the residual, see normed), norm_offset (default 0; 1: that norm's stored
+    weight is the distance from one).  names: weight, and norm where there is one."""
     graph_safe = True
 
     def tensor_specs(self):
-        return {self.names["weight"]: TensorSpec((self.params["vocab"], self.params["width"]))}
+        specs = {self.names["weight"]: TensorSpec((self.params["vocab"], self.params["width"]))}
+        if self.params.get("norm_eps") is not None:
+            specs[self.names["norm"]] = TensorSpec((self.params["width"],))
+        return specs
 
     def bind(self, tensors, rt):
         self.rt = rt
@@ -32,6 +37,16 @@ class Embedding(Part):
         if base is not None:
             exponents = torch.arange((d + 1) // 2, dtype=torch.float64) * (-2.0 / d)
             self.turns = (float(base) ** exponents / (2.0 * math.pi)).to(rt.device)
+        self.norm_w = None
+        if self.params.get("norm_eps") is not None:
+            self.norm_w = (tensors[self.names["norm"]].double() + float(self.params.get("norm_offset", 0.0))).float().contiguous()
+
+    def normed(self, rows):
+        """(residual, pending delta) for the first layer: without a norm the rows are the residual; with one the residual
+        starts from the normed rows inside the kernel of the first layer's own norm."""
+        if self.norm_w is None:
+            return rows, None
+        return torch.empty_like(rows), Joining([Term(rows, gamma=self.norm_w, eps=float(self.params["norm_eps"]))], fresh=True)
 
     @property
     def positional(self):

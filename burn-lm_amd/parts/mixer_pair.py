@@ -83,15 +83,15 @@ class MixerPair(Mixer):
             mine = m.forward_terms(x, step, v)
             if gamma is not None and (len(mine) != 1 or mine[0].row is not None or mine[0].gamma is not None or mine[0].scale != 1.0):
                 raise ValueError("mixer pair: an output norm stands behind a mixer that hands on one plain result")
-            terms += [Term(t.y, t.scale * scale, t.row, gamma, self.eps) for t in mine]
+            terms += [Term(t.y, t.scale * scale, t.row, gamma, self.eps, t.bias) for t in mine]
         return terms
 
     def forward(self, x, step, view):
         out = torch.zeros(1, x.shape[0], self.params["width"], dtype=torch.float32, device=x.device)
         terms = self.forward_terms(x, step, view)
         if self.norms[0] is not None:
-            self.rt.ops.post_norm(out[0], [(t.y, t.scale, t.gamma, t.eps) for t in terms])
+            self.rt.ops.post_norm(out[0], [(t.y, t.scale, t.gamma, t.eps, t.bias) for t in terms])
             return out
         chans = [torch.full((out.shape[2],), t.scale, dtype=torch.float32, device=x.device) for t in terms]
-        self.rt.ops.scaled_add(out[0], [(t.y, c, t.row) for t, c in zip(terms, chans)])
+        self.rt.ops.scaled_add(out[0], [(t.summed(), c, t.row) for t, c in zip(terms, chans)])
         return out

@@ -57,6 +57,6 @@ def join(rt, h, delta, out, gamma=None, eps=0.0, rows=None, write_h=True):
     """The kernel of a Joining: it joins h, and out (or None) takes the rows, normed with gamma and eps or as they are."""
     if any(t.row is not None for t in delta.terms):
         raise ValueError("results that are normed before they join the residual have no factor per token")
-    return rt.ops.post_norm(h, [(t.y, t.scale, t.gamma, t.eps) for t in delta.terms],
+    return rt.ops.post_norm(h, [(t.y, t.scale, t.gamma, t.eps, t.bias) for t in delta.terms],
                             post=None if delta.gamma is None else (delta.gamma, delta.eps), fresh=delta.fresh, vec=delta.vec,
                             write_h=write_h, gamma=gamma, eps=eps, out=out, rows=rows)

@@ -147,7 +147,7 @@ class LayerScale(Part):
         """h += sum over roles and their terms of coefficient(role, term.scale) * term.row * term.y, in float32."""
         if any(t.gamma is not None for _, ts in by_role for t in ts):
             raise ValueError("layer scale adds plain summands; results with norms of their own need a block that joins them")
-        terms = [(t.y, self.coefficient(role, t.scale), t.row) for role, ts in by_role for t in ts]
+        terms = [(t.summed(), self.coefficient(role, t.scale), t.row) for role, ts in by_role for t in ts]
         limit = self.rt.ops.MAX_ADD_TERMS
         for at in range(0, len(terms), limit):
             self.rt.ops.scaled_add(h, terms[at:at + limit])

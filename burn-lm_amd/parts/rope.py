@@ -11,6 +11,10 @@ into that order when it imports them (nn/llama/import.rs:94-127).  ``pairing="ha
 ``(i, i + head_dim/2)`` instead, which is the same function on un-permuted Hugging Face rows,
 so such checkpoints load without a re-layout.
 
+``yarn`` (default none; factor, original, fast, slow): frequencies whose pairs make more than ``fast`` turns over the
+``original`` context stay, those of fewer than ``slow`` are divided by ``factor``, with a linear ramp over the pairs between,
+and cosines and sines are multiplied by ``0.1 ln(factor) + 1`` (the table holds the product).
+
 ``rotary_dim`` (default: all of head_dim) turns only the first that many lanes of every head, with
 ``theta_i = theta^(-2i/rotary_dim)``, and passes the rest through: the table holds angle zero for
 their pairs, so the kernels need not know (pairs of "half" are then ``(i, i + rotary_dim/2)``).
@@ -44,9 +48,19 @@ def rope_frequencies(head_dim, theta, scaling=None, rotary_dim=None):
     return f
 
 
+def yarn_frequencies(head_dim, theta, factor, original, fast, slow):
+    """(frequencies float64 [head_dim/2], factor on cosines and sines)."""
+    f = rope_frequencies(head_dim, theta)
+    pair_of = lambda turns: head_dim * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(theta))
+    lo, hi = max(math.floor(pair_of(fast)), 0), min(math.ceil(pair_of(slow)), head_dim - 1)
+    ramp = np.clip((np.arange(head_dim // 2) - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return f / factor * ramp + f * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
+
+
 class RotaryEncoding(PositionEncoding):
     """params: head_dim, theta, scaling (None or 4 numbers), pairing ("half" | "interleaved"),
-    rotary_dim (optional: the lanes of a head that turn, an even number up to head_dim)."""
+    rotary_dim (optional: the lanes of a head that turn, an even number up to head_dim), yarn (optional: factor, original,
+    fast, slow; with every lane turning and no other scaling)."""
     graph_safe = True
 
 
@@ -59,7 +73,13 @@ class RotaryEncoding(PositionEncoding):
         self.rotary_dim = int(self.params.get("rotary_dim") or self.head_dim)
         if self.rotary_dim % 2 or not 2 <= self.rotary_dim <= self.head_dim or self.head_dim % 2:
             raise ValueError(f"rotary_dim must be an even number from 2 to head_dim = {self.head_dim}, got {self.rotary_dim}")
-        self.freqs = rope_frequencies(self.head_dim, self.params["theta"], self.params.get("scaling"), self.rotary_dim)
+        self.amplitude = 1.0      # factor on cosines and sines
+        if self.params.get("yarn") is not None:
+            if self.params.get("scaling") is not None or self.rotary_dim != self.head_dim:
+                raise ValueError("rotary encoding: yarn comes without another scaling and with every lane of a head turning")
+            self.freqs, self.amplitude = yarn_frequencies(self.head_dim, self.params["theta"], *self.params["yarn"])
+        else:
+            self.freqs = rope_frequencies(self.head_dim, self.params["theta"], self.params.get("scaling"), self.rotary_dim)
         self._shared = {"table": None, "n_positions": 0}    # one table for this encoding and its adjacent-pair twin
         self._twin = None
 
@@ -68,7 +88,7 @@ class RotaryEncoding(PositionEncoding):
 
     def prepare(self, n_positions, rt):
         ang = np.arange(n_positions, dtype=np.float64)[:, None] * self.freqs[None, :]
-        cs = np.stack([np.cos(ang), np.sin(ang)], axis=-1).astype(np.float32)
+        cs = (np.stack([np.cos(ang), np.sin(ang)], axis=-1) * self.amplitude).astype(np.float32)
         self._shared["table"] = torch.from_numpy(cs).to(rt.device)
         self._shared["n_positions"] = n_positions
 

@@ -187,3 +187,51 @@ class GroupedRoutedExperts(RoutedExperts):
         out = torch.zeros(1, x.shape[0], x.shape[1], dtype=torch.float32, device=x.device)
         self.rt.ops.scaled_add(out[0], [(t.y, None, t.row) for t in terms])
         return out
+
+
+class TableExperts(RoutedExperts):
+    """The same stacked experts without a router: a stored table ``[vocab, top]`` names every token id's experts (the
+    entries of a row differ), each with the weight ``1 / top``.  The step's token ids are read on the device, also those
+    that a decode step's host has not seen yet.
+
+    params: width, vocab, experts, top, expert_inner.  names: table, e<i>.gate / e<i>.up / e<i>.down."""
+
+    def tensor_specs(self):
+        p, n = self.params, self.names
+        d, f = p["width"], p["expert_inner"]
+        specs = {n["table"]: TensorSpec((p["vocab"], p["top"]), "int")}
+        for e in range(p["experts"]):
+            specs[n[f"e{e}.gate"]] = TensorSpec((f, d))
+            specs[n[f"e{e}.up"]] = TensorSpec((f, d))
+            specs[n[f"e{e}.down"]] = TensorSpec((d, f))
+        return specs
+
+    def bind(self, tensors, rt):
+        self.rt = rt
+        p, n = self.params, self.names
+        self.E, self.top, self.f, self.s = p["experts"], p["top"], p["expert_inner"], 0
+        if not 1 <= self.top <= self.E:
+            raise ValueError(f"top = {self.top} of {self.E} experts")
+        self.table = tensors[n["table"]].contiguous()
+        if int(self.table.min()) < 0 or int(self.table.max()) >= self.E:
+            raise ValueError(f"the table {n['table']} names experts outside 0 .. {self.E - 1}")
+        gates, ups, downs = ([tensors[n[f"e{e}.{r}"]] for e in range(self.E)] for r in ("gate", "up", "down"))
+        if len({w.dtype for w in gates + ups + downs}) != 1:
+            gates, ups, downs = ([w.float() for w in group] for group in (gates, ups, downs))
+        self.inner = self.E * self.f
+        self.w_gate_up = rt.weight(torch.cat(gates + ups, dim=0))
+        self.w_down = rt.weight(torch.cat(downs, dim=1).contiguous())
+
+    def step_bytes(self, rows):
+        return sum(w.w.numel() * w.w.element_size() for w in (self.w_gate_up, self.w_down)) + 4 * self.top * rows
+
+    def step_flops(self, rows):
+        return 2 * rows * sum(w.w.numel() for w in (self.w_gate_up, self.w_down))
+
+    def forward(self, x, step):
+        rt = self.rt
+        weights = torch.empty(x.shape[0], self.E + 1, dtype=torch.float32, device=x.device)
+        rt.ops.moe_table(self.table, step.token_ids, weights, self.E, step.token_source)
+        gu = rt.linear(x, self.w_gate_up)
+        act = torch.empty(x.shape[0], self.inner, dtype=gu.dtype, device=x.device)
+        return rt.linear(rt.ops.moe_gate(gu, weights, act, self.E, self.f), self.w_down, partials=True)

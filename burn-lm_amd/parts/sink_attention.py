@@ -17,7 +17,10 @@ Variants by parameter: no biases at all (``bias=False``); turning pairs of adjac
 rotation); an output gate (``gate=True``): the concatenated heads are multiplied element by element by
 ``sigmoid(W_g x)`` of the mixer's own input before the output projection (``W_g`` runs with the other projections);
 queries and keys (with their biases) divided by their root mean square over each head's lanes in front of the rotation
-(``unit_norm_eps``); capped scores ``s <- c tanh(s / c)`` (``softcap``); the first ``keep_first`` keys of a sequence visible
+(``unit_norm_eps``), or RMS-normed with stored weights over each head's lanes or over all heads' lanes together
+(``qk_norm``), without a rotation; queries that grow with their position p by ``1 + coef ln(floor((p + 1) / every) + 1)``
+(``growth``); a sink that is not learned, one added to the denominator (``sink="one"``); an output gate of one number per
+head (``gate="heads"``); capped scores ``s <- c tanh(s / c)`` (``softcap``); the first ``keep_first`` keys of a sequence visible
 beside the window, at their true positions (``keep_first``; their pages stay in the cache)."""
 from __future__ import annotations
 
@@ -36,10 +39,12 @@ class SinkAttention(Mixer):
     the default: lane i turns with lane i + rot_dims/2; "adjacent": lane 2i with 2i + 1), values ("projected", the
     default, or "keys": the unrotated keys are the values and there is no value projection), temperature (whether a
     number per head multiplies its scores; default False), gate (whether the heads pass a sigmoid gate projected from
-    the input; default False), output_bias (whether the output projection has a bias; default: as the others),
-    unit_norm_eps (default none: no norm of queries and keys), softcap (default 0: none), keep_first (default 0; first
+    the input; default False; "heads": one number per head), output_bias (whether the output projection has a bias; default: as the others),
+    unit_norm_eps (default none: no norm of queries and keys), qk_norm (default none; "heads": an RMS norm per head with a
+    weight of dim lanes for all heads; "rows": over the whole projection with a weight of all its rows; with norm_eps),
+    growth (default none; (coef, every), with qk_norm), sink "one" (the denominator holds one more, nothing is stored), softcap (default 0: none), keep_first (default 0; first
     keys that stay visible beside a window).
-    names: q, q_bias, o, o_bias, sink, talk, temp, g and, unless the layer borrows, k, k_bias, v, v_bias (those the
+    names: q, q_bias, o, o_bias, sink, talk, temp, g, q_norm, k_norm and, unless the layer borrows, k, k_bias, v, v_bias (those the
     parameters leave)."""
     graph_safe = True
 
@@ -63,14 +68,17 @@ class SinkAttention(Mixer):
         borrows, sink, talk = self._flags()
         bias, values_are_keys, _ = self._variant()
         specs = {n["q"]: TensorSpec((H * dk, d)), n["o"]: TensorSpec((d, H * dv))}
-        if sink:
+        if sink is True:
             specs[n["sink"]] = TensorSpec((H,))
         if talk:
             specs[n["talk"]] = TensorSpec((H, H))
         if p.get("temperature"):
             specs[n["temp"]] = TensorSpec((H,))
         if p.get("gate"):
-            specs[n["g"]] = TensorSpec((H * dv, d))
+            specs[n["g"]] = TensorSpec((H if p["gate"] == "heads" else H * dv, d))
+        if p.get("qk_norm"):
+            lanes = self.norm_lanes()
+            specs[n["q_norm"]], specs[n["k_norm"]] = TensorSpec((lanes[0],)), TensorSpec((lanes[1],))
         if not borrows:
             specs[n["k"]] = TensorSpec((G * dk, d))
             if not values_are_keys:
@@ -78,6 +86,11 @@ class SinkAttention(Mixer):
         biased = (("q", "k", "v") if bias else ()) + (("o",) if p.get("output_bias", bias) else ())
         specs.update({n[r + "_bias"]: TensorSpec(specs[n[r]].shape[:1]) for r in biased if n.get(r) in specs})
         return specs
+
+    def norm_lanes(self):
+        """Sizes of the stored weights of the queries' and the keys' norm."""
+        p = self.params
+        return (p["heads"] * p["dim"], p["kv_heads"] * p["dim"]) if p["qk_norm"] == "rows" else (p["dim"], p["dim"])
 
     def cache_need(self):
         p = self.params
@@ -105,9 +118,19 @@ class SinkAttention(Mixer):
             raise ValueError("rot_dims must be even, at most the key head size, and come with a rotary encoding")
         roles = ("q",) if self.borrows else ("q", "k") if self.values_are_keys else ("q", "k", "v")
         ws = [tensors[n[r]] for r in roles]
-        self.gated = bool(p.get("gate"))
-        if self.gated and bias:
-            raise ValueError("sink attention: an output gate comes without projection biases")
+        self.gated, self.gate_per_head = bool(p.get("gate")), p.get("gate") == "heads"
+        self.qk_norm = p.get("qk_norm")
+        if self.qk_norm not in (None, "heads", "rows"):
+            raise ValueError(f"sink attention: qk_norm={self.qk_norm!r} unknown (heads, rows)")
+        if self.qk_norm and (self.rot or self.borrows or self.values_are_keys or self.unit_norm_eps is not None or p.get("temperature")):
+            raise ValueError("sink attention: a norm with stored weights comes without a rotation, with keys and values of the layer's own")
+        if p.get("growth") and not self.qk_norm:
+            raise ValueError("sink attention: queries that grow with their position come with a norm")
+        self.growth = tuple(p["growth"]) if p.get("growth") else None
+        if self.qk_norm:
+            self.norm_eps = float(p["norm_eps"])
+            self.q_norm_w, self.k_norm_w = (tensors[n[r]].float().contiguous() for r in ("q_norm", "k_norm"))
+        self.att_heads = self.H      # heads as the attention kernels see them
         if self.gated:
             # the gate's columns start at a multiple of eight, so that rows of eight can be read from them at once
             rows = sum(w.shape[0] for w in ws)
@@ -142,7 +165,8 @@ class SinkAttention(Mixer):
             rt.ops.latent_attn_init(rt.device)     # the pieces' workspace, before any step is recorded
             rt.ops.sink_attn_mfma_init(rt.device)  # likewise: the shared memory of the form that stages pages
         self.temperature = tensors[n["temp"]].float().contiguous() if p.get("temperature") else None
-        self.sinks = tensors[n["sink"]].float().contiguous() if sink else None
+        self.sinks = torch.zeros(self.H, dtype=torch.float32, device=rt.device) if sink == "one" \
+            else tensors[n["sink"]].float().contiguous() if sink else None      # a score of zero adds exp(0) = 1
         self.talk = tensors[n["talk"]].float().contiguous() if talk else None
 
     def step_bytes(self, rows):
@@ -168,9 +192,8 @@ class SinkAttention(Mixer):
         return self.output(self.attend(self.project(x, step, view), step, view)), self.output_bias
 
     def forward_terms(self, x, step, view):
-        if self.output_bias is not None:
-            return super().forward_terms(x, step, view)
-        return [Term(self.forward_unbiased(x, step, view)[0])]
+        y, bias = self.forward_unbiased(x, step, view)
+        return [Term(y, bias=bias)]
 
     def project(self, x, step, view):
         """q (and k, v) of the step's tokens with their biases, q and k turned by position, k and v stored."""
@@ -183,26 +206,37 @@ class SinkAttention(Mixer):
         store = not self.borrows
         if store != bool(view.store):
             raise ValueError("a layer with key and value projections keeps its own pages, a borrowing layer reads another's")
+        if self.qk_norm:
+            return self._normed(qkv, step, view)
         rt.ops.qkv_prepare(qkv, self.bias_in, self.position.table if self.rot else None, self.rot, step,
                            view.block_table(step), view.k, view.v, view.page_size, self.H, self.G, self.dk, self.dv,
                            write_kv=store, adjacent=self.adjacent, values_are_keys=self.values_are_keys,
                            q_scale=self.temperature, unit_norm_eps=self.unit_norm_eps)
         return qkv
 
+    def _normed(self, qkv, step, view):
+        """Biases, norms and growth of the projected rows, keys and values stored -> the rows the attention reads."""
+        return self.rt.ops.qkv_norm(qkv, self.bias_in, self.q_norm_w, self.k_norm_w, self.norm_eps, step, view.block_table(step),
+                                    view.k, view.v, view.page_size, self.H, self.G, self.dk, self.dv,
+                                    whole_rows=self.qk_norm == "rows", growth=self.growth)
+
     def attend(self, qkv, step, view):
         """What the output projection reads: the heads' results, behind the output gate where the layer has one."""
         out = self._attend(qkv, step, view)
-        if self.gated:
+        if self.gate_per_head:
+            self.rt.ops.head_gate(out, qkv[:, self.gate_at:self.gate_at + self.H], self.dv)
+        elif self.gated:
             n = self.H * self.dv
             self.rt.ops.sigmoid_gate(out, qkv[:, self.gate_at:self.gate_at + n])
         return out
 
-    def _attend(self, qkv, step, view):
-        """Every token's queries over its sequence's visible keys -> [tokens, heads * vdim].  bfloat16 with pages of
+    def _attend(self, qkv, step, view, dtype=None):
+        """Every token's queries over its sequence's visible keys -> [tokens, heads * vdim] in dtype (default: the activation
+        dtype; float32: as the kernels sum them up).  bfloat16 with pages of
         64 keys and head sizes the matrix-core kernel takes: that kernel, its pages cut into pieces when a step
         brings so few tiles (decoding) that they would leave most of the chip idle; else the generic kernel."""
         rt = self.rt
-        out = torch.empty(qkv.shape[0], self.H * self.dv, dtype=rt.dtype, device=qkv.device)
+        out = torch.empty(qkv.shape[0], self.att_heads * self.dv, dtype=dtype or rt.dtype, device=qkv.device)
         if self.on_plain_kernels and view.page_size == 64 and qkv.stride(0) % 8 == 0 and qkv.data_ptr() % 16 == 0:
             return self._attend_plain(qkv, out, step, view)
         if self.on_matrix_cores and view.page_size == 64 and qkv.stride(0) % 8 == 0 and qkv.data_ptr() % 16 == 0 \
@@ -213,22 +247,22 @@ class SinkAttention(Mixer):
                 pages = (span + view.page_size - 1) // view.page_size
                 group_batch = int(os.environ.get("BURN_LM_AMD_SINK_GROUP_BATCH", "1"))
                 batches = -(-self.G // max(1, min(4, group_batch or 4))) if self.talk is not None else 1
-                tiles = step.n_seqs * self.G * -(-(self.H // self.G) // 16) * batches
+                tiles = step.n_seqs * self.G * -(-(self.att_heads // self.G) // 16) * batches
                 n_splits = max(1, min(pages, (4 * rt.compute_units) // max(1, tiles),
-                                      rt.ops.sink_attn_mfma_max_splits(step.n_seqs, 1, self.H, self.G, self.dv,
+                                      rt.ops.sink_attn_mfma_max_splits(step.n_seqs, 1, self.att_heads, self.G, self.dv,
                                                                        self.talk is not None)))
             return rt.ops.sink_attn_mfma(qkv, out, self.sinks, self.talk, step, view.block_table(step), view.k, view.v,
-                                         view.page_size, self.H, self.G, self.dk, self.dv, self.scale, self.window,
+                                         view.page_size, self.att_heads, self.G, self.dk, self.dv, self.scale, self.window,
                                          n_splits=n_splits, group_batch=group_batch)
         return rt.ops.sink_attn(qkv, out, self.sinks, self.talk, step, view.block_table(step), view.k, view.v,
-                                view.page_size, self.H, self.G, self.dk, self.dv, self.scale, self.window,
+                                view.page_size, self.att_heads, self.G, self.dk, self.dv, self.scale, self.window,
                                 keep_first=self.keep_first, softcap=self.softcap)
 
     def _attend_plain(self, qkv, out, step, view):
         """The plain attention's kernels (decode: key ranges cut as that mixer cuts them), with the sink."""
         from .attention import decode_splits
         rt, table = self.rt, view.block_table(step)
-        H, G, hd = self.H, self.G, self.dk
+        H, G, hd = self.att_heads, self.G, self.dk
         if step.max_new == 1:
             span = step.max_len_after if not self.window else min(step.max_len_after, self.window + view.page_size)
             pages = (span + view.page_size - 1) // view.page_size + -(-self.keep_first // view.page_size)

@@ -19,6 +19,7 @@ from __future__ import annotations
 
 import hashlib
 import json
+import math
 import os
 from dataclasses import dataclass
 from typing import Optional
@@ -113,6 +114,14 @@ class IntegerTable:
     layout: str = "int"
 
 
+@dataclass(frozen=True)
+class DistinctRows:
+    """Rows of different integers in [0, n) (at most n columns), kept as int32: entry j of a row is (a + j s) mod n with a
+    first entry a and a step s of the row's own, s without a common factor with n."""
+    n: int
+    layout: str = "int"
+
+
 ROLES = {"matrix": Normal(), "table": Normal(layout="table"), "norm": Ones()}
 
 
@@ -142,6 +151,16 @@ def make_tensor(name, shape, init, seed, std=0.02, norm_jitter=0.0, dtype=torch.
         chunk = CHUNK[torch.device(device).type]
         parts = [uniform_integers(key, a, min(chunk, n - a), init.n, device) for a in range(0, n, chunk)]
         return torch.cat(parts).reshape(shape).to(torch.int32)
+    if isinstance(init, DistinctRows):
+        rows, columns = shape
+        if columns > init.n:
+            raise ValueError(f"random weights: {name} asks for {columns} different integers below {init.n}")
+        key = tensor_key(seed, name)
+        steps = torch.tensor([s for s in range(1, init.n + 1) if math.gcd(s, init.n) == 1], dtype=torch.int64, device=device)
+        first = uniform_integers(key, 0, rows, init.n, device)
+        step = steps[uniform_integers(key, rows, rows, steps.numel(), device)]
+        j = torch.arange(columns, dtype=torch.int64, device=device)
+        return ((first[:, None] + j[None, :] * step[:, None]) % init.n).to(torch.int32)
     layout = getattr(init, "layout", "matrix")
     if override is not None:
         init = override
@@ -165,7 +184,7 @@ def make_tensor(name, shape, init, seed, std=0.02, norm_jitter=0.0, dtype=torch.
         scale, offset = float(std if init.std is None else init.std), 0.0
     else:
         raise ValueError(f"random weights: {name} has the initialiser {init!r}, which is none of "
-                         f"Normal, Ones, Uniform, Range, IntegerTable or a role name")
+                         f"Normal, Ones, Uniform, Range, IntegerTable, DistinctRows or a role name")
     if quick:
         g = torch.Generator(device=device)
         g.manual_seed(tensor_key(seed, name) & 0x7FFFFFFF)
