@@ -398,9 +398,25 @@ def belelorn_config(width, ff, heads, layers, vocab):
                 loop=dict(start=1, stop=3, times=2))
 
 
-DESIGNS = {"belelorn": belelorn_config, "fuvirax": fuvirax_config, "digasun": digasun_config, "girelix": girelix_config, "bitonex": bitonex_config}
+def netanex_config(width, ff, heads, layers, vocab):
+    """Differential attention (two maps of 64 lanes per head, values of 128), latent attention (a latent of 512 + 64 lanes, a
+    window of 1,024 rows, a sink, a scaled rotation, an output gate) and softmax attention over whole-row norms (heads of 128
+    lanes, a gate per head), in turn, queries of the first and the last in groups of four; every layer has 16 experts of 512
+    (as many weights as the Llama's feed-forward), of which a token's table row names 4."""
+    moe = dict(kind="moe", expert=dict(ff=512), router=dict(experts=16, top=4))
+    yarn = dict(factor=8.0, fast=32.0, original=4096, slow=1.0)
+    kinds = [dict(type="attention", mlp=moe, mixer=dict(heads=heads, kv_heads=heads // 4, dim=64, vdim=128, scale=0.125, diff=0.5,
+                                                        q_temp=dict(coef=0.1, every=1024))),
+             dict(type="latent_attention", mlp=moe, mixer=dict(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=512, scale=192 ** -0.5,
+                                                               mask=dict(size=1024), rot=dict(base=500000.0, dims=64, scaling=yarn))),
+             dict(type="attention_2", mlp=moe, mixer=dict(heads=heads, kv_heads=heads // 4, dim=128, vdim=128, scale=128 ** -0.5))]
+    return dict(architecture="Netanex", vocab=vocab, width=width, norm=dict(eps=1e-6), layers=[kinds[i % 3] for i in range(layers)])
+
+
+DESIGNS = {"netanex": netanex_config, "belelorn": belelorn_config, "fuvirax": fuvirax_config, "digasun": digasun_config, "girelix": girelix_config, "bitonex": bitonex_config}
 # the designs that run beside one (the Llama of equal size always does): the closest of those that were there before
-BESIDE = {"girelix": ("digasun",), "bitonex": ("girelix", "fuvirax"), "belelorn": ("girelix",)}
+BESIDE = {"girelix": ("digasun",), "bitonex": ("girelix", "fuvirax"), "belelorn": ("girelix",),
+          "netanex": ("girelix", "bitonex")}
 
 
 def mixer_rates(engine, batch, context, prefill_tokens):
@@ -433,7 +449,7 @@ def mixer_rates(engine, batch, context, prefill_tokens):
             mid, mix = m.project(x), m.scan
         elif kind == "ChannelDelta":
             mid, mix = m.project(x, step, v), m.scan
-        elif kind == "SinkAttention":
+        elif kind in ("SinkAttention", "DifferentialAttention"):
             if m.borrows:        # the lending layer's kernel is the same one
                 return
             mid, mix = m.project(x, step, v), m.attend
@@ -458,7 +474,7 @@ def mixer_rates(engine, batch, context, prefill_tokens):
             out[key + "_gbs"] = round(nbytes / sec / 1e9, 1)
             out[key + "_frac"] = round(nbytes / sec / 1e9 / HBM_PEAK_GBS, 4)
         if flops is not None:
-            peak = MFMA_PEAK["bf16"] if kind in ("Attention", "LatentAttention", "SinkAttention") else MFMA_PEAK["fp32"]
+            peak = MFMA_PEAK["bf16"] if kind in ("Attention", "LatentAttention", "SinkAttention", "DifferentialAttention") else MFMA_PEAK["fp32"]
             out[key + "_tflops"] = round(flops / sec / 1e12, 2)
             out[key + "_frac"] = round(flops / sec / peak, 4)
 
@@ -494,7 +510,7 @@ def mixer_rates(engine, batch, context, prefill_tokens):
 
 
 def run_design(args):
-    """--design fuvirax | digasun | girelix | bitonex | belelorn: prompt and decode throughput of the design at sizes that resemble a real
+    """--design fuvirax | digasun | girelix | bitonex | belelorn | netanex: prompt and decode throughput of the design at sizes that resemble a real
     model's layers (random weights), beside the Llama of equal size (and, for a design that has one, the closest earlier
     design), and the mixing kernels of all alone against their limits."""
     import torch
@@ -597,7 +613,7 @@ def main():
                          "launched kernel by kernel on a cache that is filled without a prompt step; prints its time and "
                          "no JSON line, and says on stderr where it is")
     ap.add_argument("--design", default=None, metavar="NAME",
-                    help="instead of the default measurement: prompt and decode throughput of a design (fuvirax, digasun, girelix, bitonex, belelorn) at model-like "
+                    help="instead of the default measurement: prompt and decode throughput of a design (fuvirax, digasun, girelix, bitonex, belelorn, netanex) at model-like "
                          "layer sizes beside the Llama of equal size, with the mixing kernels alone (--layers, default 6; "
                          "--sizes 1b-like,3b-like)")
     ap.add_argument("--sizes", default=None, help="with --design: which of its sizes, with commas between them")
