@@ -431,7 +431,7 @@ extern "C" int blm_latent_attn(const float* qabs, float* olat, int cache_dtype, 
 //                    four score tiles so that the eight rows a lane supplies are neighbours in the
 //                    transposed page (lat_key_of), as in this library's other matrix-core attention.
 // Fragments come straight from global memory (the pages of a sequence are shared by all its wavefronts and
-// stay in the caches); no shared memory, no barriers.  With n_splits > 1 the pages of a wavefront's columns
+// stay in the caches); no shared memory, no barriers.  With n_splits > 1 the half pages of a wavefront's columns
 // are cut into pieces whose partial results a second kernel adds up.
 // ---------------------------------------------------------------------------------------
 typedef __attribute__((ext_vector_type(8))) __bf16 lat_bf16x8;
@@ -450,9 +450,11 @@ __device__ __forceinline__ uint4 lat_keep_first(uint4 v, int n) {
   return make_uint4(w[0], w[1], w[2], w[3]);
 }
 
+// HALVES: how many 32-row halves of a page a step of the walk takes (2: whole pages, for unsplit runs; 1: a split run is cut
+// into pieces of half pages, and its blocks are single wavefronts so that they spread over the chip)
 #define LATM_WAVES 4
-template <int R, int DR>
-__global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
+template <int R, int DR, int HALVES, int WAVES>
+__global__ void __launch_bounds__(WAVES* BLM_WAVE)
     latent_attn_mfma_kernel(const bf16* __restrict__ q, float* __restrict__ olat, const int* __restrict__ cu_seqlens,
                             const int* __restrict__ lens_after, const int* __restrict__ block_table, int table_width,
                             const bf16* __restrict__ kcache, const bf16* __restrict__ vcache, int B, int H,
@@ -464,7 +466,7 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
   static_assert(R % 16 == 0 && W % 8 == 0, "latent lanes in tiles of 16, rows in pieces of 16 bytes");
   const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
   const int c = lane & 15, kg = lane >> 4;
-  const int tile_id = blockIdx.x * LATM_WAVES + wave;          // over sequences x tiles of 16 columns
+  const int tile_id = blockIdx.x * WAVES + wave;          // over sequences x tiles of 16 columns
   const int b = tile_id / tiles_per_seq, tile = tile_id - b * tiles_per_seq;
   if (b >= B) return;                                            // the last block's surplus wavefronts
   const int split = blockIdx.y;
@@ -484,10 +486,11 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
   const int max_qpos = past + last_idx / H;
   const int max_key = after - 1;
   const int min_qpos = past + (tile * 16) / H;                   // and the first one reaches furthest back
-  const int p_lo = (window > 0 && min_qpos - window + 1 > 0) ? (min_qpos - window + 1) / 64 : 0;
-  const int n_pages = max_qpos / 64 + 1 - p_lo;
-  const int per = (n_pages + n_splits - 1) / n_splits;
-  const int p_begin = p_lo + split * per, p_end = min(p_lo + n_pages, p_begin + per);
+  constexpr int ROWS = 32 * HALVES, TILES = 2 * HALVES;
+  const int u_lo = (window > 0 && min_qpos - window + 1 > 0) ? (min_qpos - window + 1) / ROWS : 0;
+  const int n_units = max_qpos / ROWS + 1 - u_lo;
+  const int per = (n_units + n_splits - 1) / n_splits;
+  const int u_begin = u_lo + split * per, u_end = min(u_lo + n_units, u_begin + per);
   const int lo = window > 0 ? qpos - window + 1 : 0;
   const int* bt = block_table + (size_t)b * table_width;
 
@@ -507,14 +510,14 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) o[dt] = lat_f32x4{0.f, 0.f, 0.f, 0.f};
 
-  for (int pi = p_begin; pi < p_end; ++pi) {
-    const int page = bt[pi];
-    const int key0 = pi * 64;
-    const bf16* kp = kcache + (size_t)page * 64 * W;
-    const bf16* vp = vcache + (size_t)page * R * 64;
-    float s[4][4];
+  for (int u = u_begin; u < u_end; ++u) {
+    const int page = bt[u * ROWS / 64];
+    const int key0 = u * ROWS, row0 = key0 & 63;
+    const bf16* kp = kcache + ((size_t)page * 64 + row0) * W;
+    const bf16* vp = vcache + (size_t)page * R * 64 + row0;
+    float s[TILES][4];
 #pragma unroll
-    for (int t = 0; t < 4; ++t) {
+    for (int t = 0; t < TILES; ++t) {
       const bf16* krow = kp + (size_t)lat_key_of(t, c) * W;
       uint4 kf[KS];
 #pragma unroll
@@ -535,14 +538,14 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
     }
     float mx = -INFINITY;
 #pragma unroll
-    for (int t = 0; t < 4; ++t)
+    for (int t = 0; t < TILES; ++t)
 #pragma unroll
       for (int r = 0; r < 4; ++r) mx = blm_max(mx, s[t][r]);
     mx = rows_max(mx);
     const float m_new = blm_max(m, mx * scale2);
     const float corr = (m == m_new) ? 1.f : __builtin_amdgcn_exp2f(m - m_new);
 #pragma unroll
-    for (int t = 0; t < 4; ++t)
+    for (int t = 0; t < TILES; ++t)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         s[t][r] = (s[t][r] == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(__builtin_fmaf(s[t][r], scale2, -m_new));
@@ -555,9 +558,9 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
       for (int r = 0; r < 4; ++r) l[r] *= corr;
     }
     m = m_new;
-    const bool tail = key0 + 63 > max_key;       // the page holds places past the data: 0 * garbage must stay 0
+    const bool tail = key0 + ROWS - 1 > max_key;       // these rows include places past the data: 0 * garbage must stay 0
 #pragma unroll
-    for (int h = 0; h < 2; ++h) {
+    for (int h = 0; h < HALVES; ++h) {
       uint4 pf;
       pf.x = f32x2_to_bf16x2_bits(s[2 * h][0], s[2 * h][1]);
       pf.y = f32x2_to_bf16x2_bits(s[2 * h][2], s[2 * h][3]);
@@ -599,39 +602,60 @@ __global__ void __launch_bounds__(LATM_WAVES* BLM_WAVE)
   }
 }
 
-// The pieces of a split run added up, one block per column (a (token, head) pair): maxima in base 2.  A piece
-// that saw nothing has sum 0, maximum -infinity and a result of zeros, and gets weight 0.
-#define LATM_MERGE_THREADS 256
+// The pieces of a split run added up, one block per column (a (token, head) pair) and 256 latent lanes: maxima in base 2.
+// A piece that saw nothing has sum 0, maximum -infinity and a result of zeros, and gets weight 0.  Every wavefront takes
+// each LATM_MERGE_WAVESth piece, four lanes of the latent per thread.
+#define LATM_MERGE_WAVES 4
+#define LATM_MERGE_LANES (4 * BLM_WAVE)
 #define LATM_MAX_PIECES 64
-__global__ void __launch_bounds__(LATM_MERGE_THREADS)
+__global__ void __launch_bounds__(LATM_MERGE_WAVES* BLM_WAVE)
     latent_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, float* __restrict__ olat,
                         const int* __restrict__ cu_seqlens, int H, int R, int tiles_per_seq, int n_splits) {
-  __shared__ float wgt[LATM_MAX_PIECES];
-  __shared__ float inv_sum;
+  __shared__ float wgt[LATM_MERGE_WAVES][LATM_MAX_PIECES];
+  __shared__ float4 sums[LATM_MERGE_WAVES][BLM_WAVE];
+  const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
   const int gcol = blockIdx.x;
   const int per_seq = tiles_per_seq * 16;
   const int b = gcol / per_seq, idx = gcol - b * per_seq;
   const int t_first = cu_seqlens[b], n_new = cu_seqlens[b + 1] - t_first;
-  if (idx >= n_new * H) return;
+  if (idx >= n_new * H) return;          // the whole block
   const int tok = idx / H, head = idx - tok * H;
-  float* orow = olat + ((size_t)(t_first + tok) * H + head) * R;
+  const int d = blockIdx.y * LATM_MERGE_LANES + lane * 4;
   const float* ml = part_ml + (size_t)gcol * n_splits * 2;
-  if (threadIdx.x < BLM_WAVE) {          // n_splits <= 64: one lane per piece
-    const bool has = (int)threadIdx.x < n_splits;
-    const float ms = has ? ml[threadIdx.x * 2] : -INFINITY, ls = has ? ml[threadIdx.x * 2 + 1] : 0.f;
-    const float M = wave_max(ls != 0.f ? ms : -INFINITY);
-    const float w = ls != 0.f ? __builtin_amdgcn_exp2f(ms - M) : 0.f;
-    const float L = wave_sum(ls * w);
-    if (has) wgt[threadIdx.x] = w;
-    if (threadIdx.x == 0) inv_sum = 1.0f / L;
-  }
+  // n_splits <= 64: one lane per piece, in every wavefront alike
+  const bool has = lane < n_splits;
+  const float ms = has ? ml[lane * 2] : -INFINITY, ls = has ? ml[lane * 2 + 1] : 0.f;
+  const float M = wave_max(ls != 0.f ? ms : -INFINITY);
+  const float w = ls != 0.f ? __builtin_amdgcn_exp2f(ms - M) : 0.f;
+  const float inv = 1.0f / wave_sum(ls * w);
+  wgt[wave][lane] = w;
   __syncthreads();
-  const float* po = part_o + (size_t)gcol * n_splits * R;
-  for (int d = threadIdx.x; d < R; d += LATM_MERGE_THREADS) {
-    float acc = 0.f;
-    for (int sp = 0; sp < n_splits; ++sp) acc = fmaf(po[(size_t)sp * R + d], wgt[sp], acc);
-    orow[d] = acc * inv_sum;
+  const float* po = part_o + (size_t)gcol * n_splits * R + d;
+  float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (d < R) {
+#pragma unroll 8
+    for (int sp = wave; sp < n_splits; sp += LATM_MERGE_WAVES) {
+      const float4 v = *reinterpret_cast<const float4*>(po + (size_t)sp * R);
+      const float f = wgt[wave][sp];
+      acc.x = fmaf(v.x, f, acc.x);
+      acc.y = fmaf(v.y, f, acc.y);
+      acc.z = fmaf(v.z, f, acc.z);
+      acc.w = fmaf(v.w, f, acc.w);
+    }
   }
+  sums[wave][lane] = acc;
+  __syncthreads();
+  if (wave != 0 || d >= R) return;
+#pragma unroll
+  for (int i = 1; i < LATM_MERGE_WAVES; ++i) {
+    const float4 v = sums[i][lane];
+    acc.x += v.x;
+    acc.y += v.y;
+    acc.z += v.z;
+    acc.w += v.w;
+  }
+  *reinterpret_cast<float4*>(olat + ((size_t)(t_first + tok) * H + head) * R + d) =
+      make_float4(acc.x * inv, acc.y * inv, acc.z * inv, acc.w * inv);
 }
 
 // the sizes the matrix-core form is built for (latent lanes, turned key lanes)
@@ -661,23 +685,27 @@ extern "C" int blm_latent_attn_mfma(const void* q, float* olat, const int* cu_se
   const long long tiles = ((long long)max_new * H + 15) / 16;
   const long long waves = (long long)B * tiles;
   BLM_REQUIRE(waves < 2147483647LL, "latent_attn_mfma: too many tiles");
-  const unsigned blocks = (unsigned)((waves + LATM_WAVES - 1) / LATM_WAVES);
   const float scale2 = scale * 1.4426950408889634f;
-  dim3 grid(blocks, (unsigned)n_splits);
+#define BLM_LATM_LAUNCH(r, d, halves, per_block)                                                                        \
+  hipLaunchKernelGGL((latent_attn_mfma_kernel<r, d, halves, per_block>),                                               \
+                     dim3((unsigned)((waves + (per_block)-1) / (per_block)), (unsigned)n_splits), dim3((per_block)*BLM_WAVE), 0, stream, \
+                     (const bf16*)q, olat, cu_seqlens, lens_after, block_table, table_width, (const bf16*)kcache,       \
+                     (const bf16*)vcache, B, H, (int)tiles, scale2, n_splits, part_o, part_ml, window, sinks)
 #define BLM_LATM_CASE(r, d)                                                                                            \
   if (R == r && Dr == d) {                                                                                             \
-    hipLaunchKernelGGL((latent_attn_mfma_kernel<r, d>), grid, dim3(LATM_WAVES * BLM_WAVE), 0, stream, (const bf16*)q,  \
-                       olat, cu_seqlens, lens_after, block_table, table_width, (const bf16*)kcache, (const bf16*)vcache, \
-                       B, H, (int)tiles, scale2, n_splits, part_o, part_ml, window, sinks);                            \
+    if (n_splits == 1) BLM_LATM_LAUNCH(r, d, 2, LATM_WAVES);                                                            \
+    else BLM_LATM_LAUNCH(r, d, 1, 1);                                                                                  \
     BLM_LAUNCH_CHECK("latent_attn_mfma");                                                                              \
     if (n_splits > 1) {                                                                                                \
-      hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)(waves * 16)), dim3(LATM_MERGE_THREADS), 0, stream, part_o, part_ml, \
-                         olat, cu_seqlens, H, R, (int)tiles, n_splits);                                                \
+      hipLaunchKernelGGL(latent_merge_kernel,                                                                          \
+                         dim3((unsigned)(waves * 16), (unsigned)((R + LATM_MERGE_LANES - 1) / LATM_MERGE_LANES)),       \
+                         dim3(LATM_MERGE_WAVES * BLM_WAVE), 0, stream, part_o, part_ml, olat, cu_seqlens, H, R, (int)tiles, n_splits); \
       BLM_LAUNCH_CHECK("latent_merge");                                                                                \
     }                                                                                                                  \
     return 0;                                                                                                          \
   }
   BLM_LATM_SIZES(BLM_LATM_CASE)
 #undef BLM_LATM_CASE
+#undef BLM_LATM_LAUNCH
   return blm_fail("latent_attn_mfma: a latent of %d + %d lanes is not among the sizes it is built for", R, Dr);
 }

@@ -25,7 +25,7 @@ import torch
 from .base import KVNeed, Mixer, TensorSpec
 
 DECODE_BLOCKS_PER_UNIT = 2     # blocks of four (token, head) wavefronts the split decode aims for per compute unit
-MFMA_MAX_PIECES = 64           # most pieces the matrix-core decode cuts a sequence's pages into
+MFMA_MAX_PIECES = 64           # most pieces the matrix-core decode cuts a sequence's half pages into
 
 
 class LatentAttention(Mixer):
@@ -166,10 +166,10 @@ class LatentAttention(Mixer):
         if qabs.dtype == torch.bfloat16:        # the matrix-core form: one wavefront per 16 (token, head) pairs
             if step.max_new == 1:
                 waves = step.n_seqs * ((H + 15) // 16)
-                pages = (seen + 63) // 64 + (1 if seen < step.max_len_after else 0)      # a window may begin inside a page
-                # up to a wavefront for every vector unit of the chip: a wavefront waits out a page's trip from memory
+                halves = (seen + 31) // 32 + (1 if seen < step.max_len_after else 0)     # a window may begin inside a half page
+                # up to a wavefront for every vector unit of the chip: a wavefront waits out a half page's trip from memory
                 # with nothing else to do, so short pieces are what shortens the step
-                n_splits = max(1, min(pages, (4 * rt.compute_units) // waves, MFMA_MAX_PIECES,
+                n_splits = max(1, min(halves, (4 * rt.compute_units) // waves, MFMA_MAX_PIECES,
                                       ops.latent_attn_mfma_max_splits(step.n_seqs, 1, H, R)))
             return ops.latent_attn_mfma(qabs, olat, view.k, view.v, step, view.block_table(step), view.page_size, H, R,
                                         dr, self.scale, n_splits, window=self.window, sinks=self.sinks)
