@@ -14,6 +14,11 @@
 // key part and of the queries' rotated parts), a small batched product per head, and the attention.
 #include "common.h"
 
+#include <type_traits>
+
+typedef __attribute__((ext_vector_type(8))) __bf16 lat_bf16x8;
+typedef __attribute__((ext_vector_type(4))) float lat_f32x4;
+
 // ---------------------------------------------------------------------------------------
 // down [T][ld_down]: R latent lanes then Dr key lanes.  q [T][ld_q], head h at h * (dn + Dr).  cos_sin [positions][half_t]
 // (cos, sin), of which the first rot/2 pairs turn lanes (i, i + rot/2) of the Dr part, or (adjacent) lanes (2i, 2i + 1).
@@ -213,6 +218,120 @@ __global__ void __launch_bounds__(256)
   }
 }
 
+// The same on the matrix cores: w bfloat16, inputs rounded to bfloat16 where they are float, K a multiple of eight, rows
+// that start at multiples of 16 bytes.  A = 16 weight rows (n), B = 16 input rows (t), 32 of K per instruction: a lane
+// ends up with four neighbouring n of one t.  Rows past T or N are read from the last one and not stored.
+__device__ __forceinline__ lat_bf16x8 hp_eight(const bf16* p) { return *reinterpret_cast<const lat_bf16x8*>(p); }
+__device__ __forceinline__ lat_bf16x8 hp_eight(const float* p) {
+  const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+  return __builtin_bit_cast(lat_bf16x8, make_uint4(f32x2_to_bf16x2_bits(a.x, a.y), f32x2_to_bf16x2_bits(a.z, a.w),
+                                                   f32x2_to_bf16x2_bits(b.x, b.y), f32x2_to_bf16x2_bits(b.z, b.w)));
+}
+
+__device__ __forceinline__ void hp_four(bf16* p, lat_f32x4 v) {
+  *reinterpret_cast<uint2*>(p) = make_uint2(f32x2_to_bf16x2_bits(v[0], v[1]), f32x2_to_bf16x2_bits(v[2], v[3]));
+}
+__device__ __forceinline__ void hp_four(float* p, lat_f32x4 v) { *reinterpret_cast<lat_f32x4*>(p) = v; }
+
+// wide: groups of four columns start at multiples of their size (the caller's strides say so)
+template <typename TO>
+__device__ __forceinline__ void hp_store(TO* row, int n, int N, lat_f32x4 v, bool wide) {
+  if (wide && n + 4 <= N) {
+    hp_four(row + n, v);
+    return;
+  }
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+    if (n + r < N) row[n + r] = from_float<TO>(v[r]);
+}
+
+// A wavefront makes 32 rows x 64 columns, a block 128 rows of the same columns.
+#define HPM_N 4
+#define HPM_T 2
+#define HPM_WAVES 4
+template <typename TI, typename TO>
+__global__ void __launch_bounds__(HPM_WAVES* BLM_WAVE)
+    head_project_mfma_kernel(const TI* __restrict__ in, long long in_row, int in_head, const bf16* __restrict__ w,
+                             TO* __restrict__ out, long long out_row, int out_head, int T, int N, int K, bool wide) {
+  const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
+  const int c = lane & 15, kg = lane >> 4;
+  const int h = blockIdx.z, n0 = blockIdx.y * (16 * HPM_N), t0 = (blockIdx.x * HPM_WAVES + wave) * (16 * HPM_T);
+  if (t0 >= T) return;
+  const bf16* wp[HPM_N];
+  const TI* ip[HPM_T];
+#pragma unroll
+  for (int i = 0; i < HPM_N; ++i) wp[i] = w + ((size_t)h * N + min(n0 + i * 16 + c, N - 1)) * K + kg * 8;
+#pragma unroll
+  for (int j = 0; j < HPM_T; ++j) ip[j] = in + (size_t)min(t0 + j * 16 + c, T - 1) * in_row + (size_t)h * in_head + kg * 8;
+  lat_f32x4 acc[HPM_T][HPM_N] = {};
+  const lat_bf16x8 none = {};
+  // 64 of K at a time (both pieces asked for before either is used), the last ones with a check
+  const auto pieces = [&](int k, auto checked) {
+    lat_bf16x8 a[2][HPM_N], b[2][HPM_T];
+#pragma unroll
+    for (int s = 0; s < 2; ++s) {
+      const int ks = k + s * 32;
+      const bool has = !decltype(checked)::value || ks + kg * 8 < K;
+#pragma unroll
+      for (int i = 0; i < HPM_N; ++i) a[s][i] = has ? hp_eight(wp[i] + ks) : none;
+#pragma unroll
+      for (int j = 0; j < HPM_T; ++j) b[s][j] = has ? hp_eight(ip[j] + ks) : none;
+    }
+#pragma unroll
+    for (int s = 0; s < 2; ++s)
+#pragma unroll
+      for (int j = 0; j < HPM_T; ++j)
+#pragma unroll
+        for (int i = 0; i < HPM_N; ++i) acc[j][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[s][i], b[s][j], acc[j][i], 0, 0, 0);
+  };
+  const int K64 = K & ~63;
+  for (int k = 0; k < K64; k += 64) pieces(k, std::false_type{});
+  if (K64 < K) pieces(K64, std::true_type{});
+#pragma unroll
+  for (int j = 0; j < HPM_T; ++j) {
+    const int t = t0 + j * 16 + c;
+    if (t >= T) continue;
+    TO* row = out + (size_t)t * out_row + (size_t)h * out_head;
+#pragma unroll
+    for (int i = 0; i < HPM_N; ++i) hp_store(row, n0 + i * 16 + kg * 4, N, acc[j][i], wide);
+  }
+}
+
+// Few rows (decoding): a block makes 16 rows x 16 columns, its wavefronts take every HPM_WAVESth piece of 32 of K and the
+// first one adds their sums up.
+#define HPM_FEW 128
+template <typename TI, typename TO>
+__global__ void __launch_bounds__(HPM_WAVES* BLM_WAVE)
+    head_project_few_mfma_kernel(const TI* __restrict__ in, long long in_row, int in_head, const bf16* __restrict__ w,
+                                 TO* __restrict__ out, long long out_row, int out_head, int T, int N, int K, bool wide) {
+  __shared__ lat_f32x4 sums[HPM_WAVES][BLM_WAVE];
+  const int wave = threadIdx.x / BLM_WAVE, lane = threadIdx.x & (BLM_WAVE - 1);
+  const int c = lane & 15, kg = lane >> 4;
+  const int h = blockIdx.z, n0 = blockIdx.x * 16, t = blockIdx.y * 16 + c;
+  const bf16* wp = w + ((size_t)h * N + min(n0 + c, N - 1)) * K + kg * 8;
+  const TI* ip = in + (size_t)min(t, T - 1) * in_row + (size_t)h * in_head + kg * 8;
+  lat_f32x4 acc = {};
+  const lat_bf16x8 none = {};
+  for (int k = wave * 32; k < K; k += 32 * HPM_WAVES * 4) {      // four pieces asked for at once
+    lat_bf16x8 a[4], b[4];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      const int ks = k + s * 32 * HPM_WAVES;
+      const bool has = ks + kg * 8 < K;
+      a[s] = has ? hp_eight(wp + ks) : none;
+      b[s] = has ? hp_eight(ip + ks) : none;
+    }
+#pragma unroll
+    for (int s = 0; s < 4; ++s) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[s], b[s], acc, 0, 0, 0);
+  }
+  sums[wave][lane] = acc;
+  __syncthreads();
+  if (wave != 0 || t >= T) return;
+#pragma unroll
+  for (int i = 1; i < HPM_WAVES; ++i) acc += sums[i][lane];
+  hp_store(out + (size_t)t * out_row + (size_t)h * out_head, n0 + kg * 4, N, acc, wide);
+}
+
 extern "C" int blm_head_project(const void* in, int in_dtype, long long in_row, int in_head, const void* w, int w_dtype,
                                 void* out, int out_dtype, long long out_row, int out_head, int T, int H, int N, int K,
                                 hipStream_t stream) {
@@ -220,6 +339,29 @@ extern "C" int blm_head_project(const void* in, int in_dtype, long long in_row, 
   dim3 grid((T + HP_TILE - 1) / HP_TILE, (N + HP_TILE - 1) / HP_TILE, H), block(256);
   BLM_REQUIRE(grid.y <= 65535, "head_project: too many columns");
   const unsigned few_blocks = (unsigned)(((long long)H * N + 3) / 4);
+  const size_t in_elem = in_dtype == BLM_F32 ? 4 : 2;
+  if (w_dtype == BLM_BF16 && K % 8 == 0 && (size_t)in_row * in_elem % 16 == 0 && (size_t)in_head * in_elem % 16 == 0 &&
+      ((size_t)in & 15) == 0 && ((size_t)w & 15) == 0) {
+    const bool wide = out_row % 4 == 0 && out_head % 4 == 0 && ((size_t)out & 15) == 0;
+#define BLM_HPM(TI, TO)                                                                                                  \
+  if (T <= HPM_FEW)                                                                                                      \
+    hipLaunchKernelGGL((head_project_few_mfma_kernel<TI, TO>), dim3((N + 15) / 16, (T + 15) / 16, H),                     \
+                       dim3(HPM_WAVES * BLM_WAVE), 0, stream, (const TI*)in, in_row, in_head, (const bf16*)w, (TO*)out,    \
+                       out_row, out_head, T, N, K, wide);                                                                 \
+  else                                                                                                                   \
+    hipLaunchKernelGGL((head_project_mfma_kernel<TI, TO>),                                                                \
+                       dim3((T + 16 * HPM_T * HPM_WAVES - 1) / (16 * HPM_T * HPM_WAVES), (N + 16 * HPM_N - 1) / (16 * HPM_N), H), \
+                       dim3(HPM_WAVES * BLM_WAVE), 0, stream, (const TI*)in, in_row, in_head, (const bf16*)w, (TO*)out,    \
+                       out_row, out_head, T, N, K, wide)
+    if (in_dtype == BLM_BF16 && out_dtype == BLM_F32) { BLM_HPM(bf16, float); }
+    else if (in_dtype == BLM_F32 && out_dtype == BLM_BF16) { BLM_HPM(float, bf16); }
+    else if (in_dtype == BLM_BF16 && out_dtype == BLM_BF16) { BLM_HPM(bf16, bf16); }
+    else if (in_dtype == BLM_F32 && out_dtype == BLM_F32) { BLM_HPM(float, float); }
+    else return blm_fail("head_project: unsupported dtypes in=%d w=%d out=%d", in_dtype, w_dtype, out_dtype);
+#undef BLM_HPM
+    BLM_LAUNCH_CHECK("head_project");
+    return 0;
+  }
 #define BLM_HP(TI, TW, TO)                                                                                       \
   if (T <= HP_FEW)                                                                                               \
     hipLaunchKernelGGL((head_project_few_kernel<TI, TW, TO>), dim3(few_blocks), block, 0, stream, (const TI*)in, \
@@ -434,9 +576,6 @@ extern "C" int blm_latent_attn(const float* qabs, float* olat, int cache_dtype, 
 // stay in the caches); no shared memory, no barriers.  With n_splits > 1 the half pages of a wavefront's columns
 // are cut into pieces whose partial results a second kernel adds up.
 // ---------------------------------------------------------------------------------------
-typedef __attribute__((ext_vector_type(8))) __bf16 lat_bf16x8;
-typedef __attribute__((ext_vector_type(4))) float lat_f32x4;
-
 __device__ __forceinline__ constexpr int lat_key_of(int t, int i) { return (t >> 1) * 32 + (i >> 2) * 8 + (t & 1) * 4 + (i & 3); }
 
 // keep the first n (0..8) bf16 of a 16-byte group, zero the rest

@@ -642,7 +642,7 @@ def test_latent_rows_that_stand_out_at_every_edge(form, dtype, decode, window):
         q = torch.zeros(step.n_tokens, H, W)
         q[..., R:] = 2.0
         olat = torch.empty(step.n_tokens, H, R, dtype=torch.float32, device=dev)
-        for splits in ((1, 3, 7) if decode else (1,)):
+        for splits in ((1, 3, 7, 14, 20) if decode else (1,)):
             if form == "matrix":
                 ops.latent_attn_mfma(q.to(dev, dtype), olat, kc, vc, step, table, ps, H, R, Dr, 0.5, splits, window=window)
             else:
@@ -650,6 +650,27 @@ def test_latent_rows_that_stand_out_at_every_edge(form, dtype, decode, window):
             want = torch.tensor([3.0 if P.visible(pos, j, window) else 0.0 for pos in ([p] if decode else range(n))])
             wrong = (olat.cpu() - want.view(-1, 1, 1)).abs().amax((1, 2)) > 5e-3
             assert not wrong.any(), (j, splits, wrong.nonzero().view(-1).tolist()[:5])
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("in_dtype,out_dtype", [(torch.bfloat16, torch.bfloat16), (torch.float32, torch.bfloat16), (torch.bfloat16, torch.float32)])
+@pytest.mark.parametrize("T", [1, 7, 16, 33, 128, 129, 300])
+@pytest.mark.parametrize("N,K,gap", [(64, 96, 32), (130, 128, 0), (16, 40, 8), (12, 24, 8), (96, 512, 64), (10, 18, 3)])
+def test_products_per_head(in_dtype, out_dtype, T, N, K, gap):
+    """Every head's product at row counts on both sides of each form's limits, K with and without a piece of less than 32,
+    columns that fill no tile, heads with lanes in between; what lies beside the results stays as it was."""
+    from burn_lm_amd.csrc import ops
+    dev, H, ld_head = "cuda", 3, N + 6
+    g = torch.Generator().manual_seed(T * 1000 + N + K)
+    x = torch.randn(T, H * (K + gap) + 8, generator=g).to(in_dtype)
+    w = (torch.randn(H, N, K, generator=g) * K ** -0.5).bfloat16()
+    out = torch.full((T, H * ld_head), 7.0, dtype=out_dtype, device=dev)
+    ops.head_project(x.to(dev), K + gap, w.to(dev), out, ld_head, K=K)
+    got = out.view(T, H, ld_head).double().cpu()
+    want = torch.stack([x[:, h * (K + gap):h * (K + gap) + K].bfloat16().double() @ w[h].double().T for h in range(H)], 1)
+    off = 2e-2 if out_dtype == torch.bfloat16 or in_dtype == torch.float32 else 1e-4
+    assert (got[..., :N] - want).abs().max() < off * (1 + want.abs().max())
+    assert (got[..., N:] == 7.0).all()
 
 
 @pytest.mark.gpu
@@ -674,7 +695,7 @@ def test_latent_kernels_against_plain_softmax(form, R, Dr, window, sinks):
     for news, pasts in (([100, 33], [0, 190]), ([1, 1], [149, 222])):
         step = _Step(news, pasts, dev)
         q = rt(rng.standard_normal((sum(news), H, W)))
-        for splits in ((1, 3) if step.max_new == 1 else (1,)):
+        for splits in ((1, 3, 7, 19) if step.max_new == 1 else (1,)):
             olat = torch.empty(sum(news), H, R, dtype=torch.float32, device=dev)
             if form == "matrix":
                 ops.latent_attn_mfma(q.to(dev), olat, K.to(dev), V.to(dev), step, tables, ps, H, R, Dr, scale, splits, window=window, sinks=s32)
