@@ -185,9 +185,9 @@ __global__ void __launch_bounds__(256)
 }
 
 // Queries and keys normed over their whole rows at once (all heads together).  grid (tokens, 3): the queries' part of
-// the row, the keys', the values'; a block per part.
+// the row, the keys', the values'; a block per part (of 256 threads, or of 1,024 where few tokens leave the chip idle).
 template <typename TA>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(1024)
     qkv_row_norm_kernel(TA* __restrict__ qkv, int ld, const float* __restrict__ bias, const int* __restrict__ positions,
                         const int* __restrict__ token_seq, const int* __restrict__ block_table, int table_width,
                         TA* __restrict__ kcache, TA* __restrict__ vcache, int page_size, int H, int G, int dk, int dv,
@@ -245,7 +245,7 @@ extern "C" int blm_qkv_norm(void* qkv, int dtype, int ld, const float* bias, con
   BLM_REQUIRE(every >= 0, "qkv_norm: queries that grow every %d tokens", every);
   const QnExtra ex{qw, kw, coef, every, maps, ld_q, q_out};
 #define QN_ROWS(TA)                                                                                                       \
-  hipLaunchKernelGGL(qkv_row_norm_kernel<TA>, dim3(T, 3), dim3(256), 0, stream, (TA*)qkv, ld, bias, positions, token_seq, \
+  hipLaunchKernelGGL(qkv_row_norm_kernel<TA>, dim3(T, 3), dim3(T <= 64 ? 1024 : 256), 0, stream, (TA*)qkv, ld, bias, positions, token_seq, \
                      block_table, table_width, (TA*)kcache, (TA*)vcache, page_size, H, G, dk, dv, norm_eps, ex)
 #define QN_HEADS(TA)                                                                                                      \
   hipLaunchKernelGGL(qkv_unit_kernel<TA>, dim3(T, (n_heads + 3) / 4), dim3(256), 0, stream, (TA*)qkv, ld, bias, positions, \
